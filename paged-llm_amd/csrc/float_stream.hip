@@ -8,9 +8,10 @@ using namespace pllm;
 
 // ---------------------------------------------------------------------------------------------
 // x[t, :] = float(table[ids[t], :]) * scale;  rows[t, :] = T(x[t, :]) when asked for.
+// kept: a second copy of x for whoever needs the embedding's output later (x becomes the stream that layers add to).
 template <typename T>
 __global__ void embed_scaled_kernel(const int* __restrict__ ids, const T* __restrict__ table, float* __restrict__ x,
-                                    T* __restrict__ rows, int hidden, int vocab, float scale) {
+                                    T* __restrict__ rows, float* __restrict__ kept, int hidden, int vocab, float scale) {
   const int t = blockIdx.x;
   int id = ids[t];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);  // the host has checked the range; never fault
@@ -19,17 +20,18 @@ __global__ void embed_scaled_kernel(const int* __restrict__ ids, const T* __rest
     const float v = to_f32(src[i]) * scale;
     x[(size_t)t * hidden + i] = v;
     if (rows) rows[(size_t)t * hidden + i] = from_f32<T>(v);
+    if (kept) kept[(size_t)t * hidden + i] = v;
   }
 }
 
-PLLM_API int pllm_embed_scaled(int dtype, const int* ids, const void* table, float* x, void* rows, int num_tokens,
+PLLM_API int pllm_embed_scaled(int dtype, const int* ids, const void* table, float* x, void* rows, float* kept, int num_tokens,
                                int hidden, int vocab, float scale, hipStream_t stream) {
   if (num_tokens <= 0) return 0;
   dim3 grid(num_tokens), block(256);
   if (dtype == PLLM_F32)
-    hipLaunchKernelGGL(embed_scaled_kernel<float>, grid, block, 0, stream, ids, (const float*)table, x, (float*)rows, hidden, vocab, scale);
+    hipLaunchKernelGGL(embed_scaled_kernel<float>, grid, block, 0, stream, ids, (const float*)table, x, (float*)rows, kept, hidden, vocab, scale);
   else
-    hipLaunchKernelGGL(embed_scaled_kernel<bf16>, grid, block, 0, stream, ids, (const bf16*)table, x, (bf16*)rows, hidden, vocab, scale);
+    hipLaunchKernelGGL(embed_scaled_kernel<bf16>, grid, block, 0, stream, ids, (const bf16*)table, x, (bf16*)rows, kept, hidden, vocab, scale);
   PLLM_RETURN_LAST_ERROR();
 }
 
@@ -373,6 +375,184 @@ __global__ __launch_bounds__(kHeldThreads) void rms_sandwich_held_kernel(const f
   }
 }
 
+// The same kernel where a weighted sum over the depth of the model stands behind the layer: with r = stream[row] + mult *
+// norm(branch), the layer's result,
+//   history[count][row] = r;   stream[row] = sum over j < count of depth_w[j] * history[j][row], in order, + depth_w[count] * r,
+// and `rows` are computed from that.  history holds count + 1 planes of rows, `plane` floats apart, the first `count` of
+// them filled.  The planes' rows are asked for before anything else (nothing in front of the sum needs them, and they are most of
+// what the kernel reads); VEC elements of a row lie side by side in a thread.
+struct DepthSum {
+  float* history; long plane; const float* weights; int count;
+};
+constexpr int kDepthAhead = 4;            // planes whose rows are asked for at once
+
+template <typename TO, typename TH, int VEC>
+__global__ __launch_bounds__(kHeldThreads) void rms_depth_kernel(const float* __restrict__ branch, const ChoiceSum sum, const DepthSum depth,
+                                                                 const float* __restrict__ bias, const float* __restrict__ w_branch, float mult,
+                                                                 float* __restrict__ stream, const float* __restrict__ w_next, float eps,
+                                                                 TO* __restrict__ rows, long rows_stride, int hidden, int groups) {
+  __shared__ float scratch[16];
+  constexpr int G = kHeldPerThread / VEC;
+  const int r = blockIdx.x, tid = threadIdx.x;
+  float* s = stream + (size_t)r * hidden;
+  float f[kHeldPerThread], sv[kHeldPerThread], acc[kHeldPerThread];
+  // element e of group j of this thread; groups: how many hold elements of the row at all (the rest is skipped)
+  auto at = [&](int j) { return (kHeldThreads * j + tid) * VEC; };
+  auto load = [&](const float* p, float* v) {
+    if (VEC == 4) {
+      const float4 q = *reinterpret_cast<const float4*>(p);
+      v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
+    } else {
+      v[0] = p[0];
+    }
+  };
+#pragma unroll
+  for (int i = 0; i < kHeldPerThread; ++i) f[i] = sv[i] = acc[i] = 0.f;
+#pragma unroll
+  for (int j = 0; j < G; ++j)
+    if (j < groups && at(j) < hidden) {
+      load(s + at(j), sv + j * VEC);
+      if (!sum.expert_out) load(branch + (size_t)r * hidden + at(j), f + j * VEC);
+    }
+  for (int d0 = 0; d0 < depth.count; d0 += kDepthAhead) {
+#pragma unroll
+    for (int j = 0; j < G; ++j) {
+      if (j >= groups) break;
+      const bool in = at(j) < hidden;
+      float h[kDepthAhead][VEC];
+#pragma unroll
+      for (int u = 0; u < kDepthAhead; ++u) {
+        const float* plane = depth.history + (size_t)min(d0 + u, depth.count - 1) * depth.plane + (size_t)r * hidden;
+        load(plane + (in ? at(j) : 0), h[u]);
+      }
+#pragma unroll
+      for (int u = 0; u < kDepthAhead; ++u)
+        if (d0 + u < depth.count) {
+          const float wd = depth.weights[d0 + u];
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) acc[j * VEC + e] = fmaf(wd, h[u][e], acc[j * VEC + e]);
+        }
+    }
+  }
+  if (sum.expert_out) {
+    const TH* own = reinterpret_cast<const TH*>(sum.h) + (size_t)r * sum.ld_h;
+    for (int k = 0; k < sum.top; ++k) {
+      const int row = sum.row_of_pair[(size_t)r * sum.top + k];
+      const float wk = sum.weights[(size_t)r * sum.top + k];
+      const float* e_row = sum.expert_out + (size_t)(row >= 0 ? row : 0) * hidden;
+#pragma unroll
+      for (int j = 0; j < G; ++j)
+        if (j < groups && at(j) < hidden) {
+          float v[VEC];
+          if (row >= 0) load(e_row + at(j), v);
+          else
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) v[e] = to_f32(own[at(j) + e]);
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) f[j * VEC + e] = fmaf(wk, v[e], f[j * VEC + e]);
+        }
+    }
+  }
+  float bsq = 0.f;
+#pragma unroll
+  for (int j = 0; j < G; ++j)
+    if (j < groups && at(j) < hidden) {
+      if (bias) {
+        float v[VEC];
+        load(bias + at(j), v);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) f[j * VEC + e] += v[e];
+      }
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) bsq = fmaf(f[j * VEC + e], f[j * VEC + e], bsq);
+    }
+  const float inv = w_branch ? 1.f / sqrtf(block_sum(bsq, scratch) / (float)hidden + eps) : 1.f;
+  const float w_last = depth.weights[depth.count];
+  float* keep = depth.history + (size_t)depth.count * depth.plane + (size_t)r * hidden;
+  auto store = [&](float* p, const float* v) {
+    if (VEC == 4) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+    else p[0] = v[0];
+  };
+  float sq = 0.f;
+#pragma unroll
+  for (int j = 0; j < G; ++j)
+    if (j < groups && at(j) < hidden) {
+      float wb[VEC];
+      if (w_branch) load(w_branch + at(j), wb);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        const int i = j * VEC + e;
+        sv[i] += mult * (w_branch ? f[i] * inv * wb[e] : f[i]);
+        acc[i] = fmaf(w_last, sv[i], acc[i]);
+        sq = fmaf(acc[i], acc[i], sq);
+      }
+      store(keep + at(j), sv + j * VEC);
+      store(s + at(j), acc + j * VEC);
+    }
+  if (!rows) return;
+  TO* out = rows + (size_t)r * rows_stride;
+  const float inv_next = w_next ? 1.f / sqrtf(block_sum(sq, scratch) / (float)hidden + eps) : 1.f;
+#pragma unroll
+  for (int j = 0; j < G; ++j)
+    if (j < groups && at(j) < hidden) {
+      float wn[VEC];
+      if (w_next) load(w_next + at(j), wn);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        const float y = acc[j * VEC + e];
+        out[at(j) + e] = from_f32<TO>(w_next ? y * inv_next * wn[e] : y);
+      }
+    }
+}
+
+// branch (float rows like the stream), or expert_out and what belongs to it (a sum of experts' rows); rows of up to 4,096
+// elements.
+PLLM_API int pllm_rms_depth(int out_dtype, int h_dtype, const float* branch, const float* expert_out, const void* h, long ld_h,
+                            const int* row_of_pair, const float* weights, int top, float* history, long plane, const float* depth_w, int count,
+                            const float* bias, const float* w_branch, float mult, float* stream, const float* w_next, float eps, void* rows,
+                            long rows_stride, int num_rows, int hidden, hipStream_t stream_) {
+  if (num_rows <= 0) return 0;
+  if (hidden <= 0 || hidden > kHeldPerThread * kHeldThreads || !stream || !history || !depth_w || count < 1) return -2;
+  if (expert_out ? (!h || !row_of_pair || !weights || top <= 0) : !branch) return -2;
+  const ChoiceSum sum{expert_out, h, ld_h, row_of_pair, weights, top};
+  const DepthSum depth{history, plane, depth_w, count};
+  const uintptr_t all = (uintptr_t)branch | (uintptr_t)expert_out | (uintptr_t)history | (uintptr_t)bias | (uintptr_t)w_branch | (uintptr_t)stream | (uintptr_t)w_next;
+  const int vec = hidden % 4 == 0 && plane % 4 == 0 && all % 16 == 0 ? 4 : 1;
+  const int groups = (hidden + kHeldThreads * vec - 1) / (kHeldThreads * vec);
+#define PLLM_RD(TO, TH)                                                                                                                  \
+  do {                                                                                                                                   \
+    if (vec == 4)                                                                                                                        \
+      hipLaunchKernelGGL((rms_depth_kernel<TO, TH, 4>), dim3(num_rows), dim3(kHeldThreads), 0, stream_, branch, sum, depth, bias, w_branch, \
+                         mult, stream, w_next, eps, (TO*)rows, rows_stride, hidden, groups);                                             \
+    else                                                                                                                                 \
+      hipLaunchKernelGGL((rms_depth_kernel<TO, TH, 1>), dim3(num_rows), dim3(kHeldThreads), 0, stream_, branch, sum, depth, bias, w_branch, \
+                         mult, stream, w_next, eps, (TO*)rows, rows_stride, hidden, groups);                                             \
+  } while (0)
+  if (out_dtype == PLLM_F32) { if (h_dtype == PLLM_F32) PLLM_RD(float, float); else PLLM_RD(float, bf16); }
+  else { if (h_dtype == PLLM_F32) PLLM_RD(bf16, float); else PLLM_RD(bf16, bf16); }
+#undef PLLM_RD
+  PLLM_RETURN_LAST_ERROR();
+}
+
+// The sum over the depth alone, for rows of any length: history[count] = stream;  stream = sum_j depth_w[j] history[j] + depth_w[count] stream.
+__global__ __launch_bounds__(256) void depth_sum_kernel(float* __restrict__ stream, const DepthSum depth, size_t total) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total) return;
+  float acc = 0.f;
+  for (int j = 0; j < depth.count; ++j) acc = fmaf(depth.weights[j], depth.history[(size_t)j * depth.plane + i], acc);
+  const float r = stream[i];
+  depth.history[(size_t)depth.count * depth.plane + i] = r;
+  stream[i] = fmaf(depth.weights[depth.count], r, acc);
+}
+
+PLLM_API int pllm_depth_sum(float* stream, float* history, long plane, const float* depth_w, int count, long total, hipStream_t stream_) {
+  if (total <= 0) return 0;
+  if (!stream || !history || !depth_w || count < 0 || plane < total) return -2;
+  const DepthSum depth{history, plane, depth_w, count};
+  hipLaunchKernelGGL(depth_sum_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream_, stream, depth, (size_t)total);
+  PLLM_RETURN_LAST_ERROR();
+}
+
 template <typename TO>
 static void launch_sandwich_held(int h_dtype, const float* branch, const BranchPair& pair, const ChoiceSum& sum, const float* bias, const float* w_branch, float mult,
                                  float* stream, const float* w_next, float eps, void* rows, long rows_stride, int num_rows, int hidden,
@@ -658,5 +838,43 @@ PLLM_API int pllm_scaled_sum(int dtype, const void* a, float sa, const void* b, 
     hipLaunchKernelGGL(scaled_sum_kernel<float>, grid, block, 0, stream, (const float*)a, sa, (const float*)b, sb, (float*)out, (size_t)n);
   else
     hipLaunchKernelGGL(scaled_sum_kernel<bf16>, grid, block, 0, stream, (const bf16*)a, sa, (const bf16*)b, sb, (bf16*)out, (size_t)n);
+  PLLM_RETURN_LAST_ERROR();
+}
+
+// ---------------------------------------------------------------------------------------------
+// out[t, c] = TO(act(in[t, c])) for c < cols (row_activation in common.h), rows with a row stride each; in place when out is in.
+template <typename TI, typename TO>
+__global__ __launch_bounds__(256) void activate_rows_kernel(const TI* in, long in_stride, TO* out, long out_stride, int cols, int act,
+                                                            float p0, float p1, size_t total) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total) return;
+  const size_t t = i / cols, c = i - t * cols;
+  out[t * out_stride + c] = from_f32<TO>(row_activation(to_f32(in[t * in_stride + c]), act, p0, p1));
+}
+
+PLLM_API int pllm_activate_rows(int in_dtype, int out_dtype, const void* in, long in_stride, void* out, long out_stride, int num_rows, int cols,
+                                int act, float p0, float p1, hipStream_t stream) {
+  if (num_rows <= 0 || cols <= 0) return 0;
+  if (act < 0 || act >= PLLM_ROW_ACT_COUNT) return -2;
+  const size_t total = (size_t)num_rows * cols;
+  dim3 grid((unsigned)((total + 255) / 256)), block(256);
+#define PLLM_AR(TI, TO)                                                                                                                \
+  hipLaunchKernelGGL((activate_rows_kernel<TI, TO>), grid, block, 0, stream, (const TI*)in, in_stride, (TO*)out, out_stride, cols, act, p0, p1, total)
+  if (in_dtype == PLLM_F32) { if (out_dtype == PLLM_F32) PLLM_AR(float, float); else PLLM_AR(float, bf16); }
+  else { if (out_dtype == PLLM_F32) PLLM_AR(bf16, float); else PLLM_AR(bf16, bf16); }
+#undef PLLM_AR
+  PLLM_RETURN_LAST_ERROR();
+}
+
+// ---------------------------------------------------------------------------------------------
+// x = cap tanh(x / cap), in place: capped logits.
+__global__ __launch_bounds__(256) void cap_rows_kernel(float* x, float cap, size_t n) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) x[i] = capped_score(x[i], cap);
+}
+
+PLLM_API int pllm_cap_rows(float* x, float cap, long n, hipStream_t stream) {
+  if (n <= 0) return 0;
+  hipLaunchKernelGGL(cap_rows_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, cap, (size_t)n);
   PLLM_RETURN_LAST_ERROR();
 }

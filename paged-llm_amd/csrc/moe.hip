@@ -1,10 +1,11 @@
-// A feed-forward of routed experts: every token goes through `top` of `experts` small gated feed-forwards (and, where
-// the router says so, through pass-through experts that hand the token back), weighted by router scores.
+// A feed-forward of routed experts: every token goes through `top` of `experts` small feed-forwards, gated or plain (and,
+// where the router says so, through pass-through experts that hand the token back), weighted by router scores.
 //
 //   moe_route      per token: router outputs in float, softmax over all of them, the choice among the best groups of
-//                  neighbouring experts by score + correction, the weights = the chosen experts' plain scores;
+//                  neighbouring experts by score + correction, the weights = the chosen experts' plain scores (or: the
+//                  choice by the outputs + bias themselves, the weights = the softmax over the chosen ones);
 //   moe_align      the (token, choice) pairs sorted by expert: per expert a run of rows, cut into tiles of rows;
-//   moe_expert_gemm the experts' products over those runs: act(gate h) * (up h) from the tokens' rows, and the down
+//   moe_expert_gemm the experts' products over those runs: act(gate h) * (up h) or act(up h) from the tokens' rows, and the down
 //                  product from the activations; one tile of rows per workgroup, every row's sums in ascending k,
 //                  so a pair's result does not depend on which other pairs share its tile or in which order
 //                  (bfloat16: on the matrix cores; float32, and sizes that fit no 16-byte load: plain multiply-adds);
@@ -133,7 +134,14 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
       if (values[e] == best) { at = (float)e; break; }
     return (int)(-wave_max(-at));
   };
-  if (chooser && scoring == 1) {
+  if (chooser && scoring == 2) {
+    // the outputs with their bias are scores and choice at once; the softmax over the chosen ones follows the choice
+    for (int e = lane; e < n; e += 64) {
+      const float sc = score[e] + (correction ? correction[e] : 0.f);
+      score[e] = sc;
+      choice[e] = sc;
+    }
+  } else if (chooser && scoring == 1) {
     // scores by a sigmoid of every router output on its own
     for (int e = lane; e < n; e += 64) {
       const float sc = 1.f / (1.f + expf(-score[e]));
@@ -177,26 +185,38 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
         if (mark[e / per] != -INFINITY) choice[e] = -INFINITY;
     __syncthreads();
   }
+  float largest = 0.f, sum = 0.f;                              // scoring 2: the first choice's score, the sum of exp(score - largest)
   for (int k = 0; k < top; ++k) {
     if (chooser) {
       const int at = lowest_at(choice, n);
+      float weight = score[at];
+      if (scoring == 2) {
+        if (k == 0) largest = weight;
+        weight = expf(weight - largest);
+        sum += weight;
+      }
       if (lane == 0) {
         ids[(size_t)t * top + k] = at;
-        weights[(size_t)t * top + k] = score[at];
+        weights[(size_t)t * top + k] = weight;
         choice[at] = -INFINITY;
       }
     }
     __syncthreads();
   }
+  if (scoring == 2 && chooser && lane == 0) {
+    const float inv = 1.f / sum;
+    for (int k = 0; k < top; ++k) weights[(size_t)t * top + k] *= inv;
+  }
 }
 
-// n_all = n + extra rows of the router matrix; scoring 0: softmax over the n router outputs, 1: a sigmoid of each.
+// n_all = n + extra rows of the router matrix; scoring 0: softmax over the n router outputs, 1: a sigmoid of each, 2: the
+// choice by the outputs + correction, weights = the softmax over the chosen ones' outputs + correction.
 PLLM_API int pllm_moe_route(int dtype, const void* h, int ld, const float* router_w, const float* correction, int num_tokens, int width,
                             int n_all, int extra, int scoring, int groups, int keep, int top, int* ids, float* weights, float* extras,
                             hipStream_t stream) {
   if (num_tokens <= 0) return 0;
   const int n = n_all - extra;
-  if (extra < 0 || (extra > 0 && !extras) || scoring < 0 || scoring > 1) return -2;
+  if (extra < 0 || (extra > 0 && !extras) || scoring < 0 || scoring > 2) return -2;
   if (n <= 0 || groups <= 0 || n % groups || keep <= 0 || keep > groups || top <= 0 || top > (n / groups) * keep) return -2;
   // as many parts of the row as make 16 pieces (1, 2, 4, 8 or 16 parts), none shorter than 64 elements: by the router's
   // shape alone, so that a token's scores do not depend on the step it is in
@@ -270,17 +290,23 @@ PLLM_API int pllm_moe_align(const int* ids, int pairs, int experts, int* sorted_
 }
 
 // ---------------------------------------------------------------------------------------------
+// What a product of the experts computes (FORM): the down product of sorted rows into float rows; the first product of the
+// tokens' rows, gated (two matrices) or plain (one matrix), activated into rows of the storage type.
+enum { kFormDown = 0, kFormGated = 1, kFormPlain = 2 };
+
 // One tile of rows of one expert times 64 of the expert's weight rows, plain multiply-adds with float sums in ascending k.
-//   GATED: a[row] = rows_in[sorted_pair[row] / top] (the token's row), w = [gate; up] [experts, 2 n_out, K],
+//   kFormGated: a[row] = rows_in[sorted_pair[row] / top] (the token's row), w = [gate; up] [experts, 2 n_out, K],
 //          out[row, n] = T(act(gate . a) * (up . a));
-//   else:  a[row] = rows_in[row] (the activations, already sorted), w [experts, n_out, K], out[row, n] = float sum.
+//   kFormPlain: the same rows, w [experts, n_out, K], out[row, n] = T(act(w . a));
+//   kFormDown:  a[row] = rows_in[row] (the activations, already sorted), w [experts, n_out, K], out[row, n] = float sum.
 constexpr int kMoeCols = 64, kMoeK = 32;
 
-template <typename T, bool GATED>
+template <typename T, int FORM>
 __global__ __launch_bounds__(256) void moe_expert_gemm_kernel(const T* __restrict__ rows_in, int ld_in, const T* __restrict__ w,
                                                               const int* __restrict__ tiles, const int* __restrict__ sorted_pair, int top,
                                                               int n_out, int K, void* __restrict__ out_, int ld_out, int act,
                                                               const float* __restrict__ pair_scale) {
+  constexpr bool GATED = FORM == kFormGated, FIRST = FORM != kFormDown;      // FIRST: from the tokens' rows, activated
   __shared__ float a_s[kMoeTileRows][kMoeK + 1];
   __shared__ float w_s[(GATED ? 2 : 1) * kMoeCols][kMoeK + 1];
   __shared__ int src[kMoeTileRows];
@@ -289,7 +315,7 @@ __global__ __launch_bounds__(256) void moe_expert_gemm_kernel(const T* __restric
   if (nrows <= 0) return;
   const int n0 = blockIdx.y * kMoeCols;
   const int tid = threadIdx.x;
-  if (tid < kMoeTileRows) src[tid] = tid < nrows ? (GATED ? sorted_pair[row0 + tid] / top : row0 + tid) : -1;
+  if (tid < kMoeTileRows) src[tid] = tid < nrows ? (FIRST ? sorted_pair[row0 + tid] / top : row0 + tid) : -1;
   __syncthreads();
   const T* we = w + (size_t)expert * (GATED ? 2 : 1) * n_out * K;
   const int r = tid >> 4, cg = tid & 15;           // this thread: row r, columns cg, cg + 16, cg + 32, cg + 48
@@ -317,12 +343,13 @@ __global__ __launch_bounds__(256) void moe_expert_gemm_kernel(const T* __restric
     __syncthreads();
   }
   if (r >= nrows) return;
-  const float ps = (GATED && pair_scale) ? pair_scale[sorted_pair[row0 + r]] : 1.f;
+  const float ps = (FIRST && pair_scale) ? pair_scale[sorted_pair[row0 + r]] : 1.f;
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int col = n0 + cg + 16 * j;
     if (col >= n_out) continue;
     if (GATED) reinterpret_cast<T*>(out_)[(size_t)(row0 + r) * ld_out + col] = from_f32<T>(gate_activation(acc[j] * ps, act) * (acc2[j] * ps));
+    else if (FIRST) reinterpret_cast<T*>(out_)[(size_t)(row0 + r) * ld_out + col] = from_f32<T>(row_activation(acc[j] * ps, act));
     else reinterpret_cast<float*>(out_)[(size_t)(row0 + r) * ld_out + col] = acc[j];
   }
 }
@@ -341,11 +368,12 @@ __global__ __launch_bounds__(256) void moe_expert_gemm_kernel(const T* __restric
 typedef __attribute__((ext_vector_type(8))) __bf16 moe_bf16x8;
 typedef __attribute__((ext_vector_type(4))) float moe_floatx4;
 
-template <bool GATED, int MT, int U>
+template <int FORM, int MT, int U>
 __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __restrict__ rows_in, int ld_in, const bf16* __restrict__ w,
                                                               const int* __restrict__ tiles, const int* __restrict__ sorted_pair, int top,
                                                               int n_out, int K, void* __restrict__ out_, int ld_out, int act,
                                                               const float* __restrict__ pair_scale) {
+  constexpr bool GATED = FORM == kFormGated, FIRST = FORM != kFormDown;      // FIRST: from the tokens' rows, activated
   constexpr int W = GATED ? 2 : 1;
   const int tile = blockIdx.x;
   const int expert = tiles[3 * tile], row0 = tiles[3 * tile + 1], nrows = tiles[3 * tile + 2];
@@ -358,7 +386,7 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
 #pragma unroll
   for (int t = 0; t < MT; ++t) {
     const int row = row0 + min(t * 16 + r, nrows - 1);       // rows past the tile's last repeat it: never stored
-    const int src = GATED ? sorted_pair[row] / top : row;
+    const int src = FIRST ? sorted_pair[row] / top : row;
     a_ptr[t] = rows_in + (size_t)src * ld_in + 8 * g;
   }
   const bf16* we = w + (size_t)expert * W * n_out * K;
@@ -448,12 +476,12 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
     for (int u = 0; u < U; ++u) {
       const int col = (block0 + u) * 16 + 4 * g;
       if (col >= n_out) continue;
-      if (GATED) {
+      if (FIRST) {
         bf16* o = reinterpret_cast<bf16*>(out_) + (size_t)(row0 + row) * ld_out + col;
         const float ps = pair_scale ? pair_scale[sorted_pair[row0 + row]] : 1.f;      // a factor on the pair's input row
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          if (col + i < n_out) o[i] = from_f32<bf16>(gate_activation(acc[u][0][t][i] * ps, act) * (acc[u][W - 1][t][i] * ps));
+          if (col + i < n_out) o[i] = from_f32<bf16>(GATED ? gate_activation(acc[u][0][t][i] * ps, act) * (acc[u][W - 1][t][i] * ps) : row_activation(acc[u][0][t][i] * ps, act));
       } else {
         float* o = reinterpret_cast<float*>(out_) + (size_t)(row0 + row) * ld_out + col;
         if (col + 3 < n_out && (ld_out & 3) == 0) {
@@ -475,11 +503,12 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
 // the quarters' order and stores.  Four times the wavefronts for the same bytes.  An output is the sum of four
 // accumulators instead of one, so it may differ from the other kernels' in the last place; which kernel runs depends
 // on the step's number of pairs alone.
-template <bool GATED>
+template <int FORM>
 __global__ __launch_bounds__(256) void moe_expert_splitk_kernel(const bf16* __restrict__ rows_in, int ld_in, const bf16* __restrict__ w,
                                                                 const int* __restrict__ tiles, const int* __restrict__ sorted_pair, int top,
                                                                 int n_out, int K, void* __restrict__ out_, int ld_out, int act,
                                                                 const float* __restrict__ pair_scale) {
+  constexpr bool GATED = FORM == kFormGated, FIRST = FORM != kFormDown;      // FIRST: from the tokens' rows, activated
   constexpr int W = GATED ? 2 : 1;
   __shared__ float part[3][W][4][64];
   const int tile = blockIdx.x;
@@ -489,7 +518,7 @@ __global__ __launch_bounds__(256) void moe_expert_splitk_kernel(const bf16* __re
   const int r = lane & 15, g = lane >> 4;
   const int block0 = blockIdx.y;
   const int row = row0 + min(r, nrows - 1);                  // rows past the tile's last repeat it: never stored
-  const bf16* a_ptr = rows_in + (size_t)(GATED ? sorted_pair[row] / top : row) * ld_in + 8 * g;
+  const bf16* a_ptr = rows_in + (size_t)(FIRST ? sorted_pair[row] / top : row) * ld_in + 8 * g;
   const bf16* we = w + (size_t)expert * W * n_out * K;
   const int col_r = min(block0 * 16 + r, n_out - 1);         // outputs past the last repeat it: never stored
   const bf16* w_ptr[W];
@@ -544,12 +573,12 @@ __global__ __launch_bounds__(256) void moe_expert_splitk_kernel(const bf16* __re
   if (r >= nrows) return;
   const int col = block0 * 16 + 4 * g;
   if (col >= n_out) return;
-  if (GATED) {
+  if (FIRST) {
     bf16* o = reinterpret_cast<bf16*>(out_) + (size_t)(row0 + r) * ld_out + col;
     const float ps = pair_scale ? pair_scale[sorted_pair[row0 + r]] : 1.f;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (col + i < n_out) o[i] = from_f32<bf16>(gate_activation(acc[0][i] * ps, act) * (acc[W - 1][i] * ps));
+      if (col + i < n_out) o[i] = from_f32<bf16>(GATED ? gate_activation(acc[0][i] * ps, act) * (acc[W - 1][i] * ps) : row_activation(acc[0][i] * ps, act));
   } else {
     float* o = reinterpret_cast<float*>(out_) + (size_t)(row0 + r) * ld_out + col;
 #pragma unroll
@@ -575,11 +604,12 @@ __device__ __forceinline__ void tile_barrier() {
   asm volatile("s_barrier" ::: "memory");
 }
 
-template <bool GATED>
+template <int FORM>
 __global__ __launch_bounds__(256) void moe_expert_tile_kernel(const bf16* __restrict__ rows_in, int ld_in, const bf16* __restrict__ w,
                                                               const int* __restrict__ tiles, const int* __restrict__ sorted_pair, int top,
                                                               int n_out, int K, void* __restrict__ out_, int ld_out, int act,
                                                               const float* __restrict__ pair_scale) {
+  constexpr bool GATED = FORM == kFormGated, FIRST = FORM != kFormDown;      // FIRST: from the tokens' rows, activated
   __shared__ __attribute__((aligned(16))) unsigned char lds[2][2][2][8 * 1024];   // [buffer][rows | weights][half of the k-step][8 blocks]
   const int tile = blockIdx.x;
   const int expert = tiles[3 * tile], row0 = tiles[3 * tile + 1], nrows = tiles[3 * tile + 2];
@@ -595,7 +625,7 @@ __global__ __launch_bounds__(256) void moe_expert_tile_kernel(const bf16* __rest
   for (int i = 0; i < 2; ++i) {
     const int p = tid + 256 * i, b = p >> 6, lr = (p & 63) >> 2, lg = p & 3;
     const int rr = row0 + min(b * 16 + lr, nrows - 1);       // rows past the tile's last repeat it: never stored
-    a_src[i] = rows_in + (size_t)(GATED ? sorted_pair[rr] / top : rr) * ld_in + lg * 8;
+    a_src[i] = rows_in + (size_t)(FIRST ? sorted_pair[rr] / top : rr) * ld_in + lg * 8;
     const int col = GATED ? min(n0 + (b & 3) * 16 + lr, n_out - 1) + (b >> 2) * n_out : min(n0 + b * 16 + lr, n_out - 1);
     b_src[i] = we + (size_t)col * K + lg * 8;
     put[i] = b * 1024 + (lr * 4 + (lg ^ ((lr >> 2) & 3))) * 16;
@@ -689,6 +719,16 @@ __global__ __launch_bounds__(256) void moe_expert_tile_kernel(const bf16* __rest
         for (int i = 0; i < 4; ++i)
           if (col + i < n_out) o[i] = from_f32<bf16>(gate_activation(acc[j][t][i] * ps, act) * (acc[j + 2][t][i] * ps));
       }
+    } else if (FIRST) {
+      const float ps = pair_scale ? pair_scale[sorted_pair[row0 + row]] : 1.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int col = n0 + wn * 64 + j * 16 + 4 * g;
+        bf16* o = reinterpret_cast<bf16*>(out_) + (size_t)(row0 + row) * ld_out + col;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (col + i < n_out) o[i] = from_f32<bf16>(row_activation(acc[j][t][i] * ps, act));
+      }
     } else {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
@@ -709,51 +749,62 @@ __global__ __launch_bounds__(256) void moe_expert_tile_kernel(const bf16* __rest
 
 constexpr int kSplitBelowWorkgroups = 256;                   // the compute units of the GPU this is written for
 
-template <bool GATED>
+template <int FORM>
 static void launch_moe_mfma(int tile_rows, int max_tiles, int pairs, const bf16* rows_in, int ld_in, const bf16* w, const int* tiles,
                             const int* sorted_pair, int top, int n_out, int K, void* out, int ld_out, int act, const float* pair_scale,
                             hipStream_t stream) {
+  constexpr bool GATED = FORM == kFormGated;
   const int blocks = (n_out + 15) / 16;
   if (tile_rows >= kBigRows) {
     dim3 grid(max_tiles, GATED ? (n_out + 63) / 64 : (n_out + 127) / 128);
-    hipLaunchKernelGGL((moe_expert_tile_kernel<GATED>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
+    hipLaunchKernelGGL((moe_expert_tile_kernel<FORM>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
   } else if (tile_rows >= 64) {
     constexpr int U = GATED ? 1 : 2;
     dim3 grid(max_tiles, (blocks + 4 * U - 1) / (4 * U));
-    hipLaunchKernelGGL((moe_expert_mfma_kernel<GATED, 4, U>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
+    hipLaunchKernelGGL((moe_expert_mfma_kernel<FORM, 4, U>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
   } else if ((long)min(pairs, max_tiles) * ((blocks + 3) / 4) < kSplitBelowWorkgroups && K >= 256) {
     // at most `pairs` tiles hold a row: too few workgroups of the kernel below to reach every compute unit
     dim3 grid(max_tiles, blocks);
-    hipLaunchKernelGGL((moe_expert_splitk_kernel<GATED>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
+    hipLaunchKernelGGL((moe_expert_splitk_kernel<FORM>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
   } else {
     dim3 grid(max_tiles, (blocks + 3) / 4);
-    hipLaunchKernelGGL((moe_expert_mfma_kernel<GATED, 1, 1>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
+    hipLaunchKernelGGL((moe_expert_mfma_kernel<FORM, 1, 1>), grid, dim3(256), 0, stream, rows_in, ld_in, w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale);
   }
 }
 
-// pair_scale (gated product only, or null): a factor per pair, indexed like the ids, by which the pair's input row counts
-// as multiplied (it is applied to the gate's and the up product's float sums).
+// form: kFormDown, kFormGated or kFormPlain.
+// pair_scale (first products only, or null): a factor per pair, indexed like the ids, by which the pair's input row counts
+// as multiplied (it is applied to the first products' float sums).
 // tile_rows: what moe_align was given.  Tiles of more than 16 rows are for the matrix-core kernel alone (bfloat16,
 // K and ld_in multiples of 8, 16-byte aligned operands); the plain kernel takes tiles of 16.
 // pairs: how many (token, choice) pairs the tiles hold between them (no more than that many tiles hold a row).
-PLLM_API int pllm_moe_expert_gemm(int dtype, int gated, const void* rows_in, int ld_in, const void* w, const int* tiles, int max_tiles,
+PLLM_API int pllm_moe_expert_gemm(int dtype, int form, const void* rows_in, int ld_in, const void* w, const int* tiles, int max_tiles,
                                   int tile_rows, const int* sorted_pair, int pairs, int top, int n_out, int K, void* out, int ld_out, int act,
                                   const float* pair_scale, hipStream_t stream) {
   if (max_tiles <= 0) return 0;
-  if (n_out <= 0 || K <= 0 || top <= 0 || pairs < 0 || act < 0 || act >= PLLM_ACT_COUNT) return -2;
+  if (n_out <= 0 || K <= 0 || top <= 0 || pairs < 0 || act < 0 || act >= (form == kFormPlain ? PLLM_ROW_ACT_COUNT : PLLM_ACT_COUNT) || act == PLLM_ROW_ACT_XIELU || form < kFormDown || form > kFormPlain) return -2;
   const bool matrix_cores = dtype == PLLM_BF16 && K % 8 == 0 && ld_in % 8 == 0 && ((uintptr_t)rows_in & 15) == 0 && ((uintptr_t)w & 15) == 0;
   if (tile_rows != kMoeTileRows && !(matrix_cores && (tile_rows == 64 || tile_rows == kMoeMaxTileRows))) return -2;
   if (matrix_cores) {
-    if (gated) launch_moe_mfma<true>(tile_rows, max_tiles, pairs, (const bf16*)rows_in, ld_in, (const bf16*)w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale, stream);
-    else launch_moe_mfma<false>(tile_rows, max_tiles, pairs, (const bf16*)rows_in, ld_in, (const bf16*)w, tiles, sorted_pair, top, n_out, K, out, ld_out, act, pair_scale, stream);
+#define PLLM_MOE_MFMA(F)                                                                                                          \
+  launch_moe_mfma<F>(tile_rows, max_tiles, pairs, (const bf16*)rows_in, ld_in, (const bf16*)w, tiles, sorted_pair, top, n_out, K, out, \
+                     ld_out, act, pair_scale, stream)
+    if (form == kFormGated) PLLM_MOE_MFMA(kFormGated);
+    else if (form == kFormPlain) PLLM_MOE_MFMA(kFormPlain);
+    else PLLM_MOE_MFMA(kFormDown);
+#undef PLLM_MOE_MFMA
     PLLM_RETURN_LAST_ERROR();
   }
   dim3 grid(max_tiles, (n_out + kMoeCols - 1) / kMoeCols), block(256);
 #define PLLM_MOE(T, G)                                                                                                         \
   hipLaunchKernelGGL((moe_expert_gemm_kernel<T, G>), grid, block, 0, stream, (const T*)rows_in, ld_in, (const T*)w, tiles,    \
                      sorted_pair, top, n_out, K, out, ld_out, act, pair_scale)
-  if (dtype == PLLM_F32) { if (gated) PLLM_MOE(float, true); else PLLM_MOE(float, false); }
-  else { if (gated) PLLM_MOE(bf16, true); else PLLM_MOE(bf16, false); }
+#define PLLM_MOE_FORM(T)                                                                                                      \
+  do {                                                                                                                        \
+    if (form == kFormGated) PLLM_MOE(T, kFormGated); else if (form == kFormPlain) PLLM_MOE(T, kFormPlain); else PLLM_MOE(T, kFormDown); \
+  } while (0)
+  if (dtype == PLLM_F32) PLLM_MOE_FORM(float); else PLLM_MOE_FORM(bf16);
+#undef PLLM_MOE_FORM
 #undef PLLM_MOE
   PLLM_RETURN_LAST_ERROR();
 }

@@ -161,6 +161,37 @@ def activation_code(name: str) -> int:
     return ACTIVATIONS[name]
 
 
+# of single elements, without a gate (PLLM_ROW_ACT_* in common.h); "xielu" has two parameters
+ROW_ACTIVATIONS = {**ACTIVATIONS, "gelu": 2, "xielu": 3, "tanh": 4, None: 5}
+
+
+def row_activation_code(name: str | None) -> int:
+    _need(name in ROW_ACTIVATIONS, f"activation {name!r}: one of {tuple(ROW_ACTIVATIONS)}")
+    return ROW_ACTIVATIONS[name]
+
+
+def activate_rows(rows: torch.Tensor, activation: str | None, params: tuple = (0.0, 0.0), out_dtype: torch.dtype | None = None) -> torch.Tensor:
+    """act(rows) element by element in float, contiguous [T, cols] of ``out_dtype`` (default: the rows' type); rows a view with unit
+    inner stride, either element type.  ``params``: the two numbers of "xielu" (see ``row_activation`` in common.h)."""
+    _on_gpu(rows)
+    _need(rows.dim() == 2 and rows.stride(1) == 1, "activate_rows: [T, cols] with unit inner stride")
+    out = torch.empty(rows.shape, dtype=out_dtype or rows.dtype, device=rows.device)
+    sig = [c_int, c_int, c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_int, c_float, c_float, c_void_p]
+    _check(_fn("float_stream.hip", "pllm_activate_rows", signature=sig)(
+        dtype_code(rows.dtype), dtype_code(out.dtype), _ptr(rows), rows.stride(0), _ptr(out), out.stride(0), rows.shape[0], rows.shape[1],
+        row_activation_code(activation), c_float(params[0]), c_float(params[1]), _stream()), "activate_rows")
+    return out
+
+
+def cap_rows(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """x = cap tanh(x / cap) in place, contiguous float32 (logits with a cap); returns x."""
+    _on_gpu(x)
+    _need(x.dtype == torch.float32 and x.is_contiguous() and cap > 0.0, "cap_rows takes contiguous float32 rows and a positive cap")
+    _check(_fn("float_stream.hip", "pllm_cap_rows", signature=[c_void_p, c_float, c_long, c_void_p])(_ptr(x), c_float(cap), x.numel(), _stream()),
+           "cap_rows")
+    return x
+
+
 def gate_mul(gate_up: torch.Tensor, activation: str = "silu") -> torch.Tensor:
     """[T, 2I] -> act(first half) * second half, [T, I]."""
     _on_gpu(gate_up)
@@ -1146,17 +1177,19 @@ def sigmoid_attention(q, k_pages, v_pages, block_tables, cu_seqlens_q, seq_lens_
 
 
 # ------------------------------------------------------------------------------------------- a residual stream kept in float
-def embed_scaled(ids: torch.Tensor, table: torch.Tensor, scale: float, want_rows: bool = True):
+def embed_scaled(ids: torch.Tensor, table: torch.Tensor, scale: float, want_rows: bool = True, kept: torch.Tensor | None = None):
     """(x, rows): x[t] = float(table[ids[t]]) * scale as float32 [T, hidden], and the same rounded to the table's type
-    (None for a float32 table, whose x already is the rows, or when ``want_rows`` is False)."""
-    _on_gpu(ids, table)
+    (None for a float32 table, whose x already is the rows, or when ``want_rows`` is False).  ``kept`` (contiguous float32
+    [T, hidden]) receives a second copy of x."""
+    _on_gpu(ids, table, kept)
     _need(ids.dtype == torch.int32 and ids.dim() == 1 and ids.is_contiguous(), "ids must be contiguous int32 [T]")
     _need(table.dim() == 2 and table.is_contiguous(), "embedding table must be contiguous [vocab, hidden]")
     T, (V, H) = ids.numel(), table.shape
     x = torch.empty((T, H), dtype=torch.float32, device=table.device)
     rows = torch.empty((T, H), dtype=table.dtype, device=table.device) if want_rows and table.dtype != torch.float32 else None
-    sig = [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p]
-    _check(_fn("float_stream.hip", "pllm_embed_scaled", signature=sig)(dtype_code(table.dtype), _ptr(ids), _ptr(table), _ptr(x), _ptr(rows),
+    _need(kept is None or (kept.dtype == torch.float32 and kept.shape == (T, H) and kept.is_contiguous()), f"kept: contiguous float32 [{T}, {H}]")
+    sig = [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p]
+    _check(_fn("float_stream.hip", "pllm_embed_scaled", signature=sig)(dtype_code(table.dtype), _ptr(ids), _ptr(table), _ptr(x), _ptr(rows), _ptr(kept),
                                                                       T, H, V, c_float(scale), _stream()), "embed_scaled")
     return x, rows
 
@@ -1413,6 +1446,96 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: 
     return out
 
 
+SCAN_STATE_MAX = 512              # state elements per channel that the selective scan takes
+
+
+def scan_state_size(n: int) -> int:
+    """The number of state elements per channel that the selective scan holds for a state of n: 8, 16 or a multiple of 32
+    (what is padded has A = B = C = 0 and stays zero)."""
+    return 8 if n <= 8 else 16 if n <= 16 else -(-n // 32) * 32
+
+
+def scan_chunk(max_q_len: int, num_tokens: int, channels: int) -> int:
+    """Tokens per chunk of the selective scan (0: every sequence token by token)."""
+    if max_q_len < SCAN_CHUNKS_FROM:
+        return 0
+    for limit, chunk in ((1024, 16), (4096, 32), (16384, 64)):
+        if num_tokens <= limit:
+            return chunk
+    return 128
+
+
+SCAN_CHUNKS_FROM = 128            # tokens of the longest sequence of a step from which its scans run in chunks
+
+
+def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, bc: torch.Tensor, a2: torch.Tensor, skip: torch.Tensor,
+                   z: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, seq_starts: torch.Tensor, cu_seqlens: torch.Tensor,
+                   num_seqs: int, max_q_len: int = 0) -> torch.Tensor:
+    """S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,  y_c = sum_n S[c, n] C_n + skip_c x_c,  out = y silu(z), with
+    dt = softplus(raw_dt + dt_bias).  x, z [T, channels] (views of one type, unit inner stride), raw_dt contiguous float32
+    [T, channels], bc float32 [T, 2 N] (a view: B, then C), a2 float32 [N, channels] = A log2(e) transposed, N as
+    ``scan_state_size`` gives it; S float32 [N, channels] in front of ``state[slot]``; a sequence with seq_starts == 0 starts
+    from S = 0.  Returns [T, channels] in x's type.  From ``SCAN_CHUNKS_FROM`` tokens of one sequence on (``max_q_len``) the
+    sequences run in chunks side by side, which rounds differently than token by token."""
+    _on_gpu(x, raw_dt, dt_bias, bc, a2, skip, z, state, state_slots, seq_starts, cu_seqlens)
+    T, C = x.shape
+    N = a2.shape[0]
+    _need(x.stride(1) == 1 and z.shape == (T, C) and z.stride(1) == 1 and z.dtype == x.dtype, "selective_scan x, z: [T, channels] of one type, unit inner stride")
+    _need(raw_dt.dtype == torch.float32 and raw_dt.shape == (T, C) and raw_dt.is_contiguous(), f"raw_dt: contiguous float32 [{T}, {C}]")
+    _need(scan_state_size(N) == N and N <= SCAN_STATE_MAX, f"a state of {N} per channel: 8, 16 or a multiple of 32 up to {SCAN_STATE_MAX}")
+    _need(bc.dtype == torch.float32 and bc.shape == (T, 2 * N) and bc.stride(1) == 1, f"bc: float32 [{T}, {2 * N}] with unit inner stride")
+    _need(a2.dtype == torch.float32 and a2.shape == (N, C) and a2.is_contiguous(), f"a2: float32 [{N}, {C}]")
+    for t, what in ((dt_bias, "dt_bias"), (skip, "skip")):
+        _need(t.dtype == torch.float32 and t.shape == (C,) and t.is_contiguous(), f"{what}: float32 [{C}]")
+    _check_sequences(state, state_slots, seq_starts, cu_seqlens, num_seqs)
+    _need(N * C <= state.shape[1], "the scan's state does not fit the state slot")
+    out = torch.empty((T, C), dtype=x.dtype, device=x.device)
+    chunk = scan_chunk(max_q_len, T, C)
+    max_chunks = T // chunk + num_seqs if chunk else 0
+    ws_state = torch.empty((max_chunks, N * C), dtype=torch.float32, device=x.device) if chunk else None
+    ws_steps = torch.empty((max_chunks, C), dtype=torch.float32, device=x.device) if chunk else None
+    dt = torch.empty((T, C), dtype=torch.float32, device=x.device) if chunk else None
+    sig = [c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_long,
+           c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p]
+    _check(_fn("selective_scan.hip", "pllm_selective_scan", signature=sig)(
+        dtype_code(x.dtype), _ptr(x), x.stride(0), _ptr(raw_dt), _ptr(dt), _ptr(dt_bias), _ptr(bc), bc.stride(0), _ptr(a2), _ptr(skip), _ptr(z),
+        z.stride(0), _ptr(state), state.stride(0), _ptr(state_slots), _ptr(seq_starts), _ptr(cu_seqlens), _ptr(out), num_seqs, C, N, chunk,
+        max_chunks, _ptr(ws_state), _ptr(ws_steps), _stream()), "selective_scan")
+    return out
+
+
+DELTA_MAX_DIM = 256               # size of a head that the delta memory takes
+
+
+def delta_rule(rows: torch.Tensor, columns: dict, raw_w: torch.Tensor, w0: torch.Tensor, bias_a: torch.Tensor, weight: torch.Tensor, eps: float,
+               heads: int, dim: int, state: torch.Tensor, state_slots: torch.Tensor, seq_starts: torch.Tensor, cu_seqlens: torch.Tensor,
+               num_seqs: int, max_q_len: int = 0) -> torch.Tensor:
+    """A matrix memory per head: u = k / sqrt(sum(k^2) + 1e-6), w = exp(-exp(-1/2) sigmoid(raw_w + w0)), a = sigmoid(raw_a +
+    bias_a), S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T, o_t = S_t^T r; then per head o / sqrt(mean(o^2) + eps) *
+    weight * sigmoid(gate).  ``rows`` [T, ...] holds r, k, v, raw_a and the gate, heads * dim columns each, from the columns
+    ``columns`` = {"r", "k", "v", "a", "g"} on (unit inner stride); raw_w float32 [T, heads * dim]; w0, bias_a, weight float32
+    [heads * dim].  S float32 [heads, dim, dim] in front of ``state[slot]``; a sequence with seq_starts == 0 starts from
+    S = 0.  Returns [T, heads * dim] in the rows' type."""
+    _on_gpu(rows, raw_w, w0, bias_a, weight, state, state_slots, seq_starts, cu_seqlens)
+    T, C = rows.shape[0], heads * dim
+    _need(rows.dim() == 2 and rows.stride(1) == 1 and all(0 <= columns[n] and columns[n] + C <= rows.shape[1] for n in "rkvag"),
+          f"delta_rule rows: five parts of {C} columns with unit inner stride")
+    _need(0 < dim <= DELTA_MAX_DIM, f"heads of {dim}: at most {DELTA_MAX_DIM}")
+    _need(raw_w.dtype == torch.float32 and raw_w.shape == (T, C) and raw_w.stride(1) == 1, f"raw_w: float32 [{T}, {C}]")
+    for t, what in ((w0, "w0"), (bias_a, "bias_a"), (weight, "weight")):
+        _need(t.dtype == torch.float32 and t.shape == (C,) and t.is_contiguous(), f"{what}: float32 [{C}]")
+    _check_sequences(state, state_slots, seq_starts, cu_seqlens, num_seqs)
+    _need(heads * dim * dim <= state.shape[1], "the memory does not fit the state slot")
+    out = torch.empty((T, C), dtype=rows.dtype, device=rows.device)
+    sig = [c_int, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_float, c_void_p,
+           c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]
+    _check(_fn("delta_rule.hip", "pllm_delta_rule", signature=sig)(
+        dtype_code(rows.dtype), _ptr(rows), rows.stride(0), columns["r"], columns["k"], columns["v"], columns["a"], columns["g"], _ptr(raw_w),
+        raw_w.stride(0), _ptr(w0), _ptr(bias_a), _ptr(weight), c_float(eps), _ptr(state), state.stride(0), _ptr(state_slots), _ptr(seq_starts),
+        _ptr(cu_seqlens), _ptr(out), num_seqs, heads, dim, _stream()), "delta_rule")
+    return out
+
+
 GATE_ACTIVATIONS = {"silu": 0, "sigmoid": 1, None: 2}
 
 
@@ -1639,16 +1762,77 @@ class WeightedPair:
         return scaled_sum(self.first, self.first_scale, self.second, self.second_scale)
 
 
+class DepthSum:
+    """A weighted sum over the depth of the model that takes a layer's result r: history[n - 1] = r, and the stream becomes
+    sum over j < n - 1 of weights[j] history[j] + weights[n - 1] r.  ``history`` float32 [>= n, T, hidden] (contiguous; planes
+    0 .. n - 2 filled: the embedding's output and the results of the layers before), ``weights`` float32 [n]."""
+
+    def __init__(self, history: torch.Tensor, weights: torch.Tensor):
+        self.history, self.weights = history, weights
+
+    def checked(self, rows: int, width: int):
+        h, w = self.history, self.weights
+        _on_gpu(h, w)
+        _need(w.dtype == torch.float32 and w.dim() == 1 and w.numel() >= 2 and w.is_contiguous(), "depth weights: float32 [n >= 2]")
+        _need(h.dtype == torch.float32 and h.dim() == 3 and h.shape[0] >= w.numel() and tuple(h.shape[1:]) == (rows, width) and h.is_contiguous(),
+              f"the history is contiguous float32 [>= {w.numel()}, {rows}, {width}]")
+        return h, w, w.numel() - 1
+
+
+def depth_sum(stream: torch.Tensor, depth: DepthSum) -> None:
+    """The sum over the depth on its own: the stream (float32 [rows, hidden]) is the layer's result, and becomes the sum."""
+    _on_gpu(stream)
+    _need(stream.dtype == torch.float32 and stream.dim() == 2 and stream.is_contiguous(), "the stream is contiguous float32 [rows, hidden]")
+    h, w, count = depth.checked(*stream.shape)
+    _check(_fn("float_stream.hip", "pllm_depth_sum", signature=[c_void_p, c_void_p, c_long, c_void_p, c_int, c_long, c_void_p])(
+        _ptr(stream), _ptr(h), h.stride(0), _ptr(w), count, stream.numel(), _stream()), "depth_sum")
+
+
+def _rms_depth(stream, branch, depth: DepthSum, w_branch, mult, eps, w_next, out, out_dtype, bias):
+    rows, H = stream.shape
+    if H > SANDWICH_HELD_MAX or (isinstance(branch, ChoiceSum) and not branch.plain) or isinstance(branch, WeightedPair):
+        # (rows too long for the kernel that holds them in registers, or a branch with further terms: one kernel after the other)
+        rms_sandwich(stream, branch, w_branch, mult, eps, bias=bias)
+        depth_sum(stream, depth)
+        return rms_sandwich(stream, None, None, 0.0, eps, w_next=w_next, out=out, out_dtype=out_dtype) if out is not None or out_dtype is not None else None
+    _on_gpu(stream, None if isinstance(branch, ChoiceSum) else branch, w_branch, w_next, out, bias)
+    _need(stream.dtype == torch.float32 and stream.is_contiguous(), "the stream is contiguous float32 [rows, hidden]")
+    for t, what in ((w_branch, "w_branch"), (w_next, "w_next"), (bias, "bias")):
+        _need(t is None or (t.dtype == torch.float32 and t.shape == (H,) and t.is_contiguous()), f"{what} must be float32 [{H}]")
+    hist, dw, count = depth.checked(rows, H)
+    if out is None and out_dtype is not None:
+        out = torch.empty((rows, H), dtype=out_dtype, device=stream.device)
+    _need(out is None or (out.dim() == 2 and out.shape == (rows, H) and out.stride(1) == 1), f"the rows' output is [{rows}, {H}] with unit inner stride")
+    e = h = rp = wt = None
+    if isinstance(branch, ChoiceSum):
+        e, h, rp, wt = branch.checked(rows, H)
+        branch = None
+    else:
+        _need(branch.dtype == torch.float32 and branch.shape == stream.shape and branch.is_contiguous(), "a branch is contiguous float32 rows like the stream")
+    sig = [c_int, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_void_p, c_void_p,
+           c_float, c_void_p, c_void_p, c_float, c_void_p, c_long, c_int, c_int, c_void_p]
+    _check(_fn("float_stream.hip", "pllm_rms_depth", signature=sig)(
+        dtype_code(out.dtype) if out is not None else F32, dtype_code(h.dtype) if h is not None else F32, _ptr(branch), _ptr(e), _ptr(h),
+        h.stride(0) if h is not None else 0, _ptr(rp), _ptr(wt), wt.shape[1] if wt is not None else 0, _ptr(hist), hist.stride(0), _ptr(dw), count,
+        _ptr(bias), _ptr(w_branch), c_float(mult), _ptr(stream), _ptr(w_next), c_float(eps), _ptr(out), out.stride(0) if out is not None else 0,
+        rows, H, _stream()), "rms_depth")
+    return out
+
+
 def rms_sandwich(stream: torch.Tensor, branch: torch.Tensor | None, w_branch: torch.Tensor | None, mult: float, eps: float,
                  w_next: torch.Tensor | None = None, out: torch.Tensor | None = None, out_dtype: torch.dtype | None = None,
-                 bias: torch.Tensor | None = None, row_index: torch.Tensor | None = None) -> torch.Tensor | None:
+                 bias: torch.Tensor | None = None, row_index: torch.Tensor | None = None, depth: DepthSum | None = None) -> torch.Tensor | None:
     """RMS norms around a float32 residual stream, all in float.  With ``branch`` (float32 rows like the stream, or a
     ``ChoiceSum``: a weighted sum of experts' rows that the kernel forms itself):
     stream += mult * rms_norm(branch + bias) * w_branch, in place (``w_branch`` None with float32 rows: stream += mult *
     (branch + bias), the branch as it is: the sum of a pre-norm block).  Then, when ``out`` or ``out_dtype`` is given, the
     rows of the stream as it is now are returned in that type: normed and times ``w_next``, or as they are when
     ``w_next`` is None.  ``out`` may be a view with a row stride of its own (unit inner stride).  Without a branch
-    ``row_index`` (int32) picks the rows of the stream; nothing is written to the stream then."""
+    ``row_index`` (int32) picks the rows of the stream; nothing is written to the stream then.  ``depth``: between the branch's
+    sum and the rows a ``DepthSum`` takes the stream."""
+    if depth is not None:
+        _need(branch is not None and row_index is None, "a sum over the depth stands behind a branch, and no rows are picked")
+        return _rms_depth(stream, branch, depth, w_branch, mult, eps, w_next, out, out_dtype, bias)
     if isinstance(branch, WeightedPair):
         return _rms_sandwich_pair(stream, branch, w_branch, mult, eps, w_next, out, out_dtype, bias, row_index)
     _on_gpu(stream, None if isinstance(branch, ChoiceSum) else branch, w_branch, w_next, out, bias, row_index)
@@ -1870,7 +2054,8 @@ MOE_MAX_TILE_ROWS = 128
 MOE_MAX_EXPERTS = 1024
 
 
-MOE_SCORINGS = {"softmax": 0, "sigmoid": 1}
+MOE_SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}
+MOE_FORMS = {"down": 0, "gated": 1, "plain": 2}
 
 
 def moe_route(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor | None, groups: int, keep: int, top: int,
@@ -1878,7 +2063,8 @@ def moe_route(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor 
     """(ids int32 [T, top], weights float32 [T, top]): router outputs h router_w^T in float, scores by a softmax over all of
     them or (``scoring`` "sigmoid") a sigmoid of each, the ``top`` largest of score + correction among the experts of the
     ``keep`` best of ``groups`` groups of neighbours (a group's mark: its largest corrected score), weights = the chosen
-    experts' scores.  The last ``extra`` rows of ``router_w`` are no experts: their outputs come back as they are, as a
+    experts' scores.  ``scoring`` "softmax_chosen": output + correction is what the choice looks at, and the weights are the softmax
+    over the chosen experts' output + correction alone.  The last ``extra`` rows of ``router_w`` are no experts: their outputs come back as they are, as a
     third result float32 [T, extra] (further products of the same rows that ride along)."""
     _on_gpu(h, router_w, correction)
     _need(h.dim() == 2 and h.stride(1) == 1, "moe_route rows: [T, width] with unit inner stride")
@@ -1931,12 +2117,15 @@ def moe_align(ids: torch.Tensor, experts: int, tile_rows: int = MOE_TILE_ROWS) -
 
 
 def moe_expert_gemm(rows_in: torch.Tensor, w: torch.Tensor, tiles: torch.Tensor, sorted_pair: torch.Tensor, top: int, gated: bool,
-                    activation: str = "silu", tile_rows: int = MOE_TILE_ROWS, pair_scale: torch.Tensor | None = None) -> torch.Tensor:
+                    activation: str = "silu", tile_rows: int = MOE_TILE_ROWS, pair_scale: torch.Tensor | None = None, plain: bool = False) -> torch.Tensor:
     """The experts' products over the sorted pairs.  ``gated``: rows_in [T, K] are the tokens' rows, w [experts, 2 N, K]
-    holds [gate; up] per expert, the result [pairs, N] in the rows' type is act(gate . a) * (up . a) for the pair's token.
-    Else rows_in [pairs, K] are rows in sorted order, w [experts, N, K], and the result is float32 [pairs, N].
-    ``pair_scale`` (gated only; float32, one number per pair in the order of the ids): the pair's input row counts as
-    multiplied by it (the factor goes onto the gate's and the up product's float sums)."""
+    holds [gate; up] per expert, the result [pairs, N] in the rows' type is act(gate . a) * (up . a) for the pair's token;
+    ``plain``: the same rows, w [experts, N, K], the result act(w . a) (one of ``ROW_ACTIVATIONS`` without parameters).
+    Neither: rows_in [pairs, K] are rows in sorted order, w [experts, N, K], and the result is float32 [pairs, N].
+    ``pair_scale`` (an expert's first product only; float32, one number per pair in the order of the ids): the pair's input row counts as
+    multiplied by it (the factor goes onto the float sums of the expert's first products)."""
+    _need(not (gated and plain), "an expert's first product is gated or plain")
+    form, first = "gated" if gated else "plain" if plain else "down", gated or plain
     _on_gpu(rows_in, w, tiles, sorted_pair, pair_scale)
     _need(rows_in.dim() == 2 and rows_in.stride(1) == 1 and w.dim() == 3 and w.is_contiguous() and w.dtype == rows_in.dtype
           and w.shape[2] == rows_in.shape[1], f"moe_expert_gemm shapes {tuple(rows_in.shape)} x {tuple(w.shape)}")
@@ -1947,15 +2136,16 @@ def moe_expert_gemm(rows_in: torch.Tensor, w: torch.Tensor, tiles: torch.Tensor,
                                          and rows_in.stride(0) % 8 == 0), "tiles of more than 16 rows are the matrix-core kernels'")
     K = rows_in.shape[1]
     N = w.shape[1] // 2 if gated else w.shape[1]
-    _need(gated or rows_in.shape[0] == pairs, "the down product takes one row per pair")
-    _need(not gated or (w.shape[1] % 2 == 0 and rows_in.shape[0] * top == pairs), "the gated product takes the tokens' rows")
-    _need(pair_scale is None or (gated and pair_scale.dtype == torch.float32 and pair_scale.numel() == pairs and pair_scale.is_contiguous()),
-          f"pair_scale: float32 [{pairs}], for the gated product")
-    out = torch.empty((pairs, N), dtype=rows_in.dtype if gated else torch.float32, device=rows_in.device)
+    _need(first or rows_in.shape[0] == pairs, "the down product takes one row per pair")
+    _need(not first or ((w.shape[1] % 2 == 0 or not gated) and rows_in.shape[0] * top == pairs), "an expert's first product takes the tokens' rows")
+    _need(activation != "xielu", "an activation with parameters is not for experts")
+    _need(pair_scale is None or (first and pair_scale.dtype == torch.float32 and pair_scale.numel() == pairs and pair_scale.is_contiguous()),
+          f"pair_scale: float32 [{pairs}], for an expert's first product")
+    out = torch.empty((pairs, N), dtype=rows_in.dtype if first else torch.float32, device=rows_in.device)
     _check(_fn("moe.hip", "pllm_moe_expert_gemm", signature=[c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int,
                                                               c_void_p, c_int, c_int, c_void_p, c_void_p])(
-        dtype_code(rows_in.dtype), int(gated), _ptr(rows_in), rows_in.stride(0), _ptr(w), _ptr(tiles), tiles.shape[0], tile_rows, _ptr(sorted_pair), pairs, top, N, K,
-        _ptr(out), out.stride(0), activation_code(activation), _ptr(pair_scale), _stream()), "moe_expert_gemm")
+        dtype_code(rows_in.dtype), MOE_FORMS[form], _ptr(rows_in), rows_in.stride(0), _ptr(w), _ptr(tiles), tiles.shape[0], tile_rows, _ptr(sorted_pair), pairs, top, N, K,
+        _ptr(out), out.stride(0), row_activation_code(activation) if plain else activation_code(activation), _ptr(pair_scale), _stream()), "moe_expert_gemm")
     return out
 
 

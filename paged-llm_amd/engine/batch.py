@@ -71,6 +71,10 @@ class StepContext:
     # Set around a branch by a block that norms the branch's output in float before adding it: the branch's last product
     # then returns float32 rows (no rounding to the compute type between the product's sums and the norm).
     float_branch: bool = False
+    # The results of the layers so far, float32 [runs + 1, T, hidden] (plane 0: the embedding's output), in models with a sum over
+    # the depth; and the operation on the stream behind the layer under way.
+    stream_history: object = None
+    exit_op: object = None
 
     @property
     def decode_only(self) -> bool:

@@ -6,6 +6,7 @@ from __future__ import annotations
 import torch
 
 from ..cache.kv_cache import CacheGroup
+from ..csrc import ops
 from ..parts import registry
 from ..parts.base import name_under, tensor_name
 from ..parts.registry import BuildEnv
@@ -30,6 +31,15 @@ class DecoderModel:
             self.blocks.append(block)
         # operations on the stream between layers, which schedule steps name as their entry
         self.stream_ops = [registry.build("stream_op", op.part, env) for op in spec.stream_ops]
+        self._keeps_history = any(op.reads_history for op in self.stream_ops)
+        # stream operations that may read the embedding's output (x0)
+        self._reads_embedding = any(not op.reads_history for op in self.stream_ops)
+        for pos, step in enumerate(spec.schedule):
+            results = getattr(self.stream_ops[step.exit], "results", None) if step.exit is not None else None
+            if results is not None and results != pos + 2:
+                raise ValueError(f"behind schedule step {pos} there are {pos + 2} results, the operation there sums {results}")
+            if step.entry is not None and self.stream_ops[step.entry].reads_history:
+                raise ValueError(f"schedule step {pos}: an operation over the results of the layers stands behind a layer, not in front of it")
         self.final_norm = registry.build("norm", spec.final_norm, env)
         self.head = registry.build("head", spec.head, env)
         self._ready = False
@@ -124,13 +134,23 @@ class DecoderModel:
         the layers still run to fill the cache)."""
         assert self._ready, "weights not loaded"
         stateful_embedding = hasattr(self.embedding, "forward_step")
-        x = (self.embedding.forward_step(ctx, states.get(self.EMBEDDING_STATE)) if stateful_embedding
-             else self.embedding.forward(ctx.input_ids))
-        delta = None
         schedule = self.spec.schedule
+        # the results of all layers in float, for operations that sum over the depth: the embedding's output, then one plane per run
+        history = None
+        if self._keeps_history and ctx.num_tokens:
+            history = torch.empty((len(schedule) + 1, ctx.num_tokens, self.spec.hidden_size), dtype=torch.float32, device=self.device)
+        if history is not None and not stateful_embedding and getattr(self.embedding, "keeps_copy", False):
+            x = self.embedding.forward(ctx.input_ids, kept=history[0])
+        else:
+            x = (self.embedding.forward_step(ctx, states.get(self.EMBEDDING_STATE)) if stateful_embedding
+                 else self.embedding.forward(ctx.input_ids))
+            if history is not None:
+                ops.place_rows(x, history[0])
+        ctx.stream_history = history
+        delta = None
         # the embedding's output for the stream operations: a tensor of its own where the layers add to the stream in place
         x0 = None
-        if self.stream_ops:
+        if self._reads_embedding:
             if stateful_embedding:
                 x0 = self.embedding.forward_step(ctx, states.get(self.EMBEDDING_STATE), again=True)
             else:
@@ -143,6 +163,10 @@ class DecoderModel:
             # the norm that reads the stream next, for a block that can compute its rows while it forms the stream's last sum
             following = schedule[pos + 1] if pos + 1 < len(schedule) else None
             ctx.next_entry_norm = (self.blocks[following.layer].entry_norm() if following is not None and following.entry is None else None)
+            # the operation behind this layer: the block takes it into its last kernel, or it is applied below
+            ctx.exit_op = self.stream_ops[step.exit] if step.exit is not None else None
+            if ctx.exit_op is not None and not block.takes_exit_op:
+                ctx.next_entry_norm = None
             if step.entry is not None:
                 # the stream operation in front of this layer may norm for the layer in the kernel that forms its sum
                 ctx.next_entry_norm, after_op = block.entry_norm(), ctx.next_entry_norm
@@ -156,7 +180,13 @@ class DecoderModel:
             ctx.partial_sums_ok = (self.blocks[schedule[pos + 1].layer].accepts_partial_delta() if pos + 1 < len(schedule)
                                    else last_takes_partial)
             x, delta = block.forward(x, delta, ctx, cache, states.get(pos))
-        ctx.partial_sums_ok = False
+            if ctx.exit_op is not None:
+                if delta is not None:
+                    raise RuntimeError("a stream operation takes the stream with every sum done")
+                x, ctx.exit_op = ctx.exit_op.forward(x, x0, ctx), None
+            elif history is not None and step.exit is None:
+                ops.place_rows(x, history[pos + 1])                # (a run without an operation behind it: its result is kept all the same)
+        ctx.partial_sums_ok, ctx.stream_history = False, None
         n = ctx.logits_index.numel()
         if n == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=self.device)

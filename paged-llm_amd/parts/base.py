@@ -214,6 +214,9 @@ class StreamOp(Part):
     and adds to (a tensor of its own: x0 is never written to)."""
     graph_capturable = True
     graph_capturable_prompts = True
+    # True: the operation reads the results of all layers before (``ctx.stream_history`` [runs + 1, T, hidden] in float32: the
+    # embedding's output, then every run's result), which the model then keeps for the step.
+    reads_history = False
 
     def forward(self, x: torch.Tensor, x0: torch.Tensor, ctx) -> torch.Tensor:
         raise NotImplementedError
@@ -236,6 +239,9 @@ class Block(Part):
     been added yet, so that the next norm can add it in the same kernel.
     """
     ROLES: dict = {}
+    # True when the block hands ``ctx.exit_op`` (an operation on the stream behind this layer) to the kernel that forms its last
+    # sum and sets it to None; else the model applies the operation behind the block.
+    takes_exit_op = False
     # The role whose part owns the layer's cache and state (None: the layer keeps nothing).
     MIXER_ROLE: str | None = "mixer"
 
@@ -289,6 +295,9 @@ class Block(Part):
                 for name, spec in part.weight_specs().items()}
 
     def assign(self, name, tensor):
+        for part in self.parts.values():
+            if "/" + name in part.weight_specs():             # a tensor that the part names outside its prefix
+                return part.assign("/" + name, tensor)
         # (the longest prefix first: "norm1" must not take what belongs to a part named "norm1.x")
         for role, part in sorted(self.parts.items(), key=lambda rp: -len(self.names[rp[0]])):
             own = name_under(self.names[role], name)

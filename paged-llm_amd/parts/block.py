@@ -104,11 +104,13 @@ class SandwichNormBlock(Block):
     stream in place and computes, from the row it still holds, the rows that whoever reads the stream next wants: this
     block's next norm, or the first norm of the layer that follows (``ctx.next_entry_norm``, set by the model), which
     travel beside the stream in ``ctx.launch_cache``.  A branch may hand a bias of its last product to that kernel
-    (``output_bias`` of the part) instead of adding it itself.
+    (``output_bias`` of the part) instead of adding it itself.  A weighted sum over the depth behind the layer
+    (``ctx.exit_op`` with ``depth_terms``) is formed by that kernel as well, between the layer's last sum and those rows.
 
     params: ``residual_mult`` (m), ``feed_forward`` (False: the mixer alone), and the roles' prefixes in tensor names."""
     ROLES = {"mixer_norm": "norm", "mixer": "mixer", "mixer_out_norm": "norm",
              "feed_forward_norm": "norm", "feed_forward": "feed_forward", "feed_forward_out_norm": "norm"}
+    takes_exit_op = True
     _ROWS = "sandwich_rows"
 
     def __init__(self, params: dict, env):
@@ -149,7 +151,13 @@ class SandwichNormBlock(Block):
             a, bias, last = m, getattr(p["feed_forward"], "output_bias", None), p["feed_forward_out_norm"]
         else:
             last = p["mixer_out_norm"]
-        rows = last.add_to(x, a, self.mult, bias=bias, then=after, want_rows=after is not None)
+        depth = None
+        if getattr(ctx, "exit_op", None) is not None:
+            if not hasattr(ctx.exit_op, "depth_terms"):
+                after = None                      # another operation follows: whoever reads the stream behind it norms for itself
+            else:
+                depth, ctx.exit_op = ctx.exit_op.depth_terms(ctx), None
+        rows = last.add_to(x, a, self.mult, bias=bias, then=after, want_rows=after is not None, depth=depth)
         ctx.launch_cache[self._ROWS] = (x, after, rows) if after is not None else None
         ctx.float_branch = ctx.branch_bias_taken = False
         return x, None

@@ -34,9 +34,13 @@ class TokenEmbedding(Part):
             raise KeyError(name)
         self.table = tensor.to(device=self.device, dtype=self.dtype).contiguous()
 
-    def forward(self, ids: torch.Tensor) -> torch.Tensor:
+    keeps_copy = True            # ``forward(ids, kept)`` leaves a second copy of the float rows (what a sum over the depth starts with)
+
+    def forward(self, ids: torch.Tensor, kept: torch.Tensor | None = None) -> torch.Tensor:
         if self.float_stream:
-            return ops.embed_scaled(ids, self.table, self.scale, want_rows=False)[0]
+            return ops.embed_scaled(ids, self.table, self.scale, want_rows=False, kept=kept)[0]
+        if kept is not None:
+            raise RuntimeError("a copy of the embedding's output is kept in float32 (float_stream)")
         if self.scale != 1.0:
             raise NotImplementedError("a scaled embedding leaves as a float stream (float_stream)")
         return ops.embed_gather(ids, self.table)
@@ -95,7 +99,10 @@ class HashedBigramEmbedding(Part):
 
 
 class LMHead(Part):
+    """params: ``vocab_size``, ``tied``, ``tensor_name`` and ``cap`` (logits become cap tanh(logits / cap), in float; 0: none)."""
+
     def __init__(self, params: dict, env: BuildEnv):
+        self.cap = float(params.get("cap") or 0.0)
         self.vocab = int(params["vocab_size"])
         self.hidden = env.hidden_size
         self.tied = bool(params.get("tied", False))
@@ -122,7 +129,8 @@ class LMHead(Part):
     def forward(self, h) -> torch.Tensor:
         if self._matrix is None:                      # (the tiled copy for decode steps, made once the matrix is there)
             self._matrix = Weight(self.weight)
-        return linear(h, self._matrix, out_dtype=torch.float32)
+        logits = linear(h, self._matrix, out_dtype=torch.float32)
+        return ops.cap_rows(logits, self.cap) if self.cap > 0.0 else logits
 
 
 register_embedding("token_embedding", TokenEmbedding)

@@ -91,22 +91,32 @@ class RMSNorm(Norm):
     def __init__(self, params: dict, env: BuildEnv):
         """params: ``eps``; ``size`` (default: the model's width); ``weight_name`` (the weight's own name under the part's
         prefix, default "weight"; "" is the prefix itself); ``unit_offset`` (the checkpoint stores w - 1: the factor
-        applied is 1 + what is stored, formed in float when the weight arrives)."""
+        applied is 1 + what is stored, formed in float when the weight arrives); ``scale_name`` (a second vector by which the
+        normed rows are multiplied element by element, stored under that name: the scale of what a sublayer adds to the
+        stream; it becomes part of the factor)."""
         self.eps = float(params["eps"])
         self.size = int(params.get("size", env.hidden_size))
         self.weight_name = params.get("weight_name", "weight")
         self.unit_offset = bool(params.get("unit_offset", False))
+        self.scale_name = params.get("scale_name")
         self.dtype, self.device = env.dtype, env.device
         self.weight: torch.Tensor | None = None
+        self._factors: dict = {}
 
     def weight_specs(self):
-        return {self.weight_name: WeightSpec((self.size,), role="vector", init="zeros" if self.unit_offset else "ones")}
+        specs = {self.weight_name: WeightSpec((self.size,), role="vector", init="zeros" if self.unit_offset else "ones")}
+        if self.scale_name is not None:
+            specs[self.scale_name] = WeightSpec((self.size,), role="vector", init="ones")
+        return specs
 
     def assign(self, name, tensor):
-        if name != self.weight_name:
+        if name not in self.weight_specs():
             raise KeyError(name)
         w = tensor.to(device=self.device, dtype=torch.float32)
-        self.weight = (w + 1.0 if self.unit_offset else w).contiguous()
+        self._factors[name] = (w + 1.0 if name == self.weight_name and self.unit_offset else w).contiguous()
+        self.weight = self._factors.get(self.weight_name)
+        if self.weight is not None and self.scale_name in self._factors:
+            self.weight = (self.weight * self._factors[self.scale_name]).contiguous()
 
     def forward(self, x, row_index=None):
         if x.dtype == torch.float32 and self.dtype != torch.float32:        # rows of a float stream, normed into the compute type
@@ -114,14 +124,15 @@ class RMSNorm(Norm):
         return ops.rmsnorm(x, self.weight, self.eps, None, row_index)
 
     def add_to(self, stream: torch.Tensor, branch: torch.Tensor, mult: float = 1.0, bias: torch.Tensor | None = None,
-               then: "RMSNorm | None" = None, out: torch.Tensor | None = None, want_rows: bool = True):
-        """stream += mult * norm(branch + bias), in place and in float (a block that norms what its branches return).
+               then: "RMSNorm | None" = None, out: torch.Tensor | None = None, want_rows: bool = True, depth=None):
+        """stream += mult * norm(branch + bias), in place and in float (a block that norms what its branches return); with
+        ``depth`` (``ops.DepthSum``) the result then enters a weighted sum over the depth, which becomes the stream.
         Returns the new stream's rows in the compute type for whoever reads them next, computed in the same kernel:
         normed by ``then`` (the reader's own norm), or as they are; into ``out`` when given; None unless ``want_rows``."""
         if then is not None and (then.eps != self.eps or then.size != self.size):
             raise ValueError("the norm behind the sum shares this norm's width and eps")
         return ops.rms_sandwich(stream, branch, self.weight, mult, self.eps, w_next=then.weight if then is not None else None,
-                                out=out, out_dtype=self.dtype if want_rows and out is None else None, bias=bias)
+                                out=out, out_dtype=self.dtype if want_rows and out is None else None, bias=bias, depth=depth)
 
     takes_weighted_pair = True          # ``sum_then`` forms a branch that is the weighted sum of two (``ops.WeightedPair``) in its kernel
 

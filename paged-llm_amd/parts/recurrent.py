@@ -1,6 +1,6 @@
 """Mixers that carry a state of fixed size per request instead of a growing cache.
 
-Both are the same recurrence per head, S_t = a_t S_(t-1) + k_t (g_t v_t)^T, y_t = S_t^T q_t (+ skip v_t), with S
+Most are the same recurrence per head, S_t = a_t S_(t-1) + k_t (g_t v_t)^T, y_t = S_t^T q_t (+ skip v_t), with S
 [N, P] in float in the request's state slot (``ops.linear_recurrence``); they differ in where a, g, k, q and v come from:
 
 * ``mamba2`` (the state-space layer in its dual form): one input product gives a gate z, the values x, the keys B and
@@ -24,6 +24,13 @@ Both are the same recurrence per head, S_t = a_t S_(t-1) + k_t (g_t v_t)^T, y_t 
   rows of S one by one, S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T; q passes SiLU; behind it each head's output is divided by
   its root mean square, times a weight that the heads share, the output product.
 
+Two recurrences have kernels of their own:
+
+* ``mamba1`` (a selective scan, ``ops.selective_scan``): a state of N floats per channel whose decays exp(dt_c A[c, n]) differ
+  from element to element, behind a short convolution; step sizes through a low-rank product, times silu(z), the output product.
+* ``general_delta`` (``ops.delta_rule``): a matrix memory whose rows decay one by one and from which, in front of every write, a
+  part of what the unit key reads is removed along another direction; norm per head, weight, sigmoid gate, output product.
+
 What enters the recurrence (step sizes, decays, rotated keys and queries, the state) is float whatever the compute type;
 the products, the convolution and the activations run in the compute type.  A request's state is zero at its first
 token (``ctx.seq_starts == 0``), whatever its slot held before.
@@ -31,13 +38,15 @@ token (``ctx.seq_starts == 0``), whatever its slot held before.
 
 from __future__ import annotations
 
+import math
+
 import torch
 
 from ..csrc import ops
 from .base import Mixer, StateSpec
 from .linear import Weight, linear
 from .registry import BuildEnv, register_mixer
-from .spec import PartSpec, WeightSpec
+from .spec import OpenSize, PartSpec, WeightSpec
 
 
 def _out_dtype(ctx):
@@ -307,6 +316,114 @@ class Hgrn2Mixer(_StatefulMixer):
         return linear(u, self.w_o, out_dtype=_out_dtype(ctx))
 
 
+class Mamba1Mixer(_StatefulMixer):
+    """A selective scan:  [x | z] = W_in h; x passes a causal convolution per channel (with bias) and SiLU;  [low | B | C] = W_x x,
+    dt = softplus(W_dt low + b);  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n with A = -exp(A_log),
+    y_c = sum_n S[c, n] C_n + D_c x_c;  then y silu(z), the output product.  Step sizes, decays, B, C and the state are float
+    whatever the compute type.  The state slot holds S [N, inner] (N padded to a size the kernel takes, the padding zero) and
+    behind it the convolution's last inputs.
+
+    params: ``inner`` (channels), ``state`` (N), ``dt_rank``, ``conv`` (taps).  Tensors: ``in`` [2 inner, width], ``conv`` [inner,
+    taps] with ``conv.b``, ``x`` [dt_rank + 2 N, inner], ``dt`` [inner, dt_rank] with ``dt.b``, ``A_log`` [inner, N], ``D`` [inner], ``o``."""
+
+    def __init__(self, params: dict, env: BuildEnv):
+        self.hidden = env.hidden_size
+        self.inner, self.N = int(params["inner"]), int(params["state"])
+        self.rank, self.taps = int(params["dt_rank"]), int(params["conv"])
+        if not 1 <= self.taps <= ops.MAX_CONV_TAPS:
+            raise ValueError(f"the convolution kernel takes 1 to {ops.MAX_CONV_TAPS} taps, got {self.taps}")
+        if not 1 <= self.N <= ops.SCAN_STATE_MAX or self.inner <= 0 or self.rank <= 0:
+            raise ValueError(f"a selective scan takes 1 to {ops.SCAN_STATE_MAX} state elements per channel; got {self.N}, {self.inner} channels, rank {self.rank}")
+        self.dtype, self.device = env.dtype, env.device
+        self.held = ops.scan_state_size(self.N)
+        self.conv_at = self.held * self.inner
+        self._w: dict = {}
+        self.w_in = self.w_x = self.w_dt = self.w_o = self.a2 = None
+
+    def weight_specs(self):
+        C = self.inner
+        return {"in": WeightSpec((2 * C, self.hidden)), "conv": WeightSpec((C, self.taps), role="vector"), "conv.b": WeightSpec((C,), role="vector"),
+                "x": WeightSpec((self.rank + 2 * self.N, C)), "dt": WeightSpec((C, self.rank)), "dt.b": WeightSpec((C,), role="vector"),
+                "A_log": WeightSpec((C, self.N), role="vector"), "D": WeightSpec((C,), role="vector"), "o": WeightSpec((self.hidden, C))}
+
+    def finalize(self):
+        w, pad = self._w, self.held - self.N
+        self.w_in, self.w_dt, self.w_o = Weight(w.pop("in")), Weight(w.pop("dt")), Weight(w.pop("o"))
+        low, b, c = w.pop("x").split([self.rank, self.N, self.N], dim=0)
+        zeros = b.new_zeros((pad, self.inner))
+        self.w_x = Weight(torch.cat([low, b, zeros, c, zeros], dim=0).contiguous())
+        a2 = torch.zeros((self.held, self.inner), dtype=torch.float32)
+        a2[:self.N] = (-torch.exp(w.pop("A_log").double().cpu()) * math.log2(math.e)).T.float()      # A log2(e), one row per state element
+        self.a2 = a2.to(self.device).contiguous()
+
+    def state_spec(self):
+        return StateSpec((self.conv_at + self.inner * (self.taps - 1),), torch.float32)
+
+    def forward(self, h, ctx, cache, state):
+        w, C = self._w, self.inner
+        proj = linear(h, self.w_in)
+        seqs = (ctx.state_slots, ctx.seq_starts, ctx.cu_seqlens_q, ctx.num_seqs)
+        x = ops.causal_conv(proj[:, :C], w["conv"], w["conv.b"], state, self.conv_at, *seqs, ctx.max_q_len)
+        low = linear(x, self.w_x, out_dtype=torch.float32)
+        step = low[:, :self.rank]
+        if self.dtype != torch.float32:
+            step = ops.activate_rows(step, None, out_dtype=self.dtype)
+        raw = linear(step, self.w_dt, out_dtype=torch.float32)
+        y = ops.selective_scan(x, raw, w["dt.b"], low[:, self.rank:], self.a2, w["D"], proj[:, C:], state, *seqs, max_q_len=ctx.max_q_len)
+        return linear(y, self.w_o, out_dtype=_out_dtype(ctx))
+
+
+class GeneralDeltaMixer(_StatefulMixer):
+    """A generalized delta rule:  r = W_r h, k = W_k h, v = W_v h; a decay w = exp(-exp(-1/2) sigmoid(W_w2 tanh(W_w1 h) + w0)) and a
+    removal rate a = sigmoid(W_a h + b_a) per head and key channel; with the unit key u = k / sqrt(sum(k^2) + 1e-6)
+    S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T  and  o_t = S_t^T r;  then each head's o divided by its root mean
+    square, times ``norm`` (over all heads' channels), times sigmoid(W_g h), the output product.  Decays, rates, unit keys, the
+    state and the norm are float whatever the compute type.
+
+    params: ``heads``, ``dim`` (of a head's keys and values), ``eps``, ``decay_rank`` (inner size of the decay's product for random
+    weights; a checkpoint's tensors decide it).  Tensors ``r``, ``k``, ``v``, ``a``, ``g`` [heads dim, width], ``a.b``, ``w0``, ``norm``
+    [heads dim], ``w1`` [rank, width], ``w2`` [heads dim, rank], ``o`` [width, heads dim]."""
+
+    def __init__(self, params: dict, env: BuildEnv):
+        self.hidden = env.hidden_size
+        self.heads, self.dim, self.eps = int(params["heads"]), int(params["dim"]), float(params["eps"])
+        self.rank = OpenSize(params.get("decay_rank") or 64)
+        if not 1 <= self.dim <= ops.DELTA_MAX_DIM or self.heads <= 0:
+            raise ValueError(f"the delta memory takes heads of 1 to {ops.DELTA_MAX_DIM}; got {self.heads} heads of {self.dim}")
+        self.dtype, self.device = env.dtype, env.device
+        self._w: dict = {}
+        self.w_in = self.w_w2 = self.w_o = None
+
+    def weight_specs(self):
+        C = self.heads * self.dim
+        specs = {n: WeightSpec((C, self.hidden)) for n in ("r", "k", "v", "a", "g")}
+        specs.update({n: WeightSpec((C,), role="vector") for n in ("a.b", "w0")})
+        specs.update({"w1": WeightSpec((self.rank, self.hidden)), "w2": WeightSpec((C, self.rank)),
+                      "norm": WeightSpec((C,), role="vector", init="ones"), "o": WeightSpec((self.hidden, C))})
+        return specs
+
+    def finalize(self):
+        w, C = self._w, self.heads * self.dim
+        if w["w1"].shape[0] != w["w2"].shape[1]:
+            raise ValueError(f"the decay's product does not fit: w1 {tuple(w['w1'].shape)}, w2 {tuple(w['w2'].shape)}")
+        self.w_in = Weight(torch.cat([w.pop(n) for n in ("r", "k", "v", "a", "g", "w1")], dim=0).contiguous())
+        self.w_w2, self.w_o = Weight(w.pop("w2")), Weight(w.pop("o"))
+        self.columns = {n: i * C for i, n in enumerate(("r", "k", "v", "a", "g"))}
+
+    def state_spec(self):
+        return StateSpec((self.heads * self.dim * self.dim,), torch.float32)
+
+    def forward(self, h, ctx, cache, state):
+        w, C = self._w, self.heads * self.dim
+        rows = linear(h, self.w_in)
+        raw_w = linear(ops.activate_rows(rows[:, 5 * C:], "tanh"), self.w_w2, out_dtype=torch.float32)
+        u = ops.delta_rule(rows, self.columns, raw_w, w["w0"], w["a.b"], w["norm"], self.eps, self.heads, self.dim, state,
+                           ctx.state_slots, ctx.seq_starts, ctx.cu_seqlens_q, ctx.num_seqs, max_q_len=ctx.max_q_len)
+        return linear(u, self.w_o, out_dtype=_out_dtype(ctx))
+
+
+register_mixer("mamba1", Mamba1Mixer)
+register_mixer("general_delta", GeneralDeltaMixer)
 register_mixer("lightning", LightningMixer)
 register_mixer("hgrn2", Hgrn2Mixer)
 register_mixer("mamba2", Mamba2Mixer)

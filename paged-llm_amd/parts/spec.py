@@ -22,9 +22,13 @@ class PartSpec:
         return json.dumps([self.kind, self.params], sort_keys=True, default=str)
 
 
+class OpenSize(int):
+    """A size that no configuration gives: the checkpoint's tensor decides it.  The number itself is what random weights take."""
+
+
 @dataclass
 class WeightSpec:
-    """One tensor a part expects from the checkpoint.
+    """One tensor a part expects from the checkpoint.  A dimension of ``shape`` that is an ``OpenSize`` may have any size.
 
     role "matrix"/"table": kept in the compute type (bfloat16 or float32).
     role "vector": kept in float32 (norm weights are applied in float).
@@ -55,10 +59,12 @@ class ScheduleStep:
     A layer named by several steps shares its weights between them; each step still owns a
     cache and a state of its own, because what it sees differs.  ``cache_from`` names an earlier
     step whose cache this step's mixer reads instead of writing one.  ``entry`` names a stream operation of the model
-    (an index into ``ModelSpec.stream_ops``) that acts on the residual stream right before this step's layer."""
+    (an index into ``ModelSpec.stream_ops``) that acts on the residual stream right before this step's layer, ``exit`` one
+    that acts on it right behind the layer."""
     layer: int
     cache_from: int | None = None
     entry: int | None = None
+    exit: int | None = None
 
 
 @dataclass
@@ -105,6 +111,8 @@ class ModelSpec:
                 raise ValueError(f"schedule step {pos} names layer {step.layer}, the model has {len(self.layers)}")
             if step.entry is not None and not 0 <= step.entry < len(self.stream_ops):
                 raise ValueError(f"schedule step {pos} names stream operation {step.entry}, the model has {len(self.stream_ops)}")
+            if step.exit is not None and not 0 <= step.exit < len(self.stream_ops):
+                raise ValueError(f"schedule step {pos} names stream operation {step.exit}, the model has {len(self.stream_ops)}")
             src = step.cache_from
             if src is not None:
                 if not 0 <= src < pos:

@@ -1,4 +1,5 @@
-"""Operations on the residual stream between layers (family "stream_op").
+"""Operations on the residual stream between layers (family "stream_op"), named by schedule steps: in front of the step's
+layer (``entry``) or behind it (``exit``).
 
 ``concat_projection``: x <- W [x ; x0], one product over the stream and the embedding's output side by side (W is
 [width, 2 width], the stream's columns first).  The operands are the two rows in the compute type, the result is a
@@ -71,3 +72,42 @@ class AddEmbedding(StreamOp):
 
 
 register_stream_op("add_embedding", AddEmbedding)
+
+
+class DepthAverage(StreamOp):
+    """x <- sum over j <= i + 1 of weights[j] X_j behind layer i, with X_0 the embedding's output and X_(j + 1) the result of
+    layer j before this operation, all in float: every layer's result reaches every later layer with a weight of its own.
+    The results are kept for the step in ``ctx.stream_history``; a block whose kernel forms the layer's last sum may take the
+    operation into it (``depth_terms``).
+
+    params: ``results`` (i + 2, how many weights there are), ``tensor_name`` (their own name under the part's prefix; "" is the
+    prefix itself)."""
+    reads_history = True
+
+    def __init__(self, params: dict, env: BuildEnv):
+        self.results = int(params["results"])
+        if self.results < 2:
+            raise ValueError(f"behind a layer there are at least two results (the embedding's output and the layer's own), got {self.results}")
+        self.tensor_name = params.get("tensor_name", "weight")
+        self.device = env.device
+        self.weights: torch.Tensor | None = None
+
+    def weight_specs(self):
+        return {self.tensor_name: WeightSpec((self.results,), role="vector", init="ones")}
+
+    def assign(self, name, tensor):
+        if name != self.tensor_name:
+            raise KeyError(name)
+        self.weights = tensor.to(device=self.device, dtype=torch.float32).contiguous()
+
+    def depth_terms(self, ctx):
+        return ops.DepthSum(ctx.stream_history, self.weights)
+
+    def forward(self, x, x0, ctx):
+        if x.dtype != torch.float32:
+            raise RuntimeError("the results of the layers are kept and summed in float32 (an embedding with float_stream)")
+        ops.depth_sum(x, self.depth_terms(ctx))
+        return x
+
+
+register_stream_op("depth_average", DepthAverage)

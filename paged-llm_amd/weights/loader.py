@@ -1,6 +1,7 @@
 """Weights from ``*.safetensors`` by tensor name (pagedllm/model/loader.py:39-69).
 
-Every tensor the model declares must be present with the declared shape, and nothing else may
+Every tensor the model declares must be present with the declared shape (a dimension the part leaves open, an ``OpenSize``,
+may have any size), and nothing else may
 be present (apart from names the spec says to ignore, and a tied head stored a second time).
 All problems are collected and reported in one ``WeightsError`` that lists missing and
 unexpected tensors and wrong shapes.  Tensors are read one at a time and handed to the part that
@@ -14,6 +15,8 @@ import glob
 import os
 
 import torch
+
+from ..parts.spec import OpenSize
 
 
 class WeightsError(KeyError):
@@ -51,13 +54,17 @@ def checkpoint_index(model_dir: str) -> dict:
     return index
 
 
+def _fits(shape, expected) -> bool:
+    return len(shape) == len(expected) and all((int(a) > 0) if isinstance(b, OpenSize) else a == b for a, b in zip(shape, expected))
+
+
 def check_names_and_shapes(expected: dict, optional: dict, ignored_suffixes: tuple, found: dict, where: str) -> None:
     """``expected``/``optional``: name -> shape; ``found``: name -> shape."""
     missing = sorted(n for n in expected if n not in found)
     unexpected, wrong = [], []
     for name, shape in sorted(found.items()):
         if name in expected:
-            if tuple(shape) != tuple(expected[name]):
+            if not _fits(tuple(shape), tuple(expected[name])):
                 wrong.append((name, tuple(shape), tuple(expected[name])))
         elif name in optional:
             if tuple(shape) != tuple(optional[name]):
