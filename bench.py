@@ -261,6 +261,58 @@ def run_renadra(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
     return out
 
 
+def mekusun_config(width: int, vocab: int) -> dict:
+    """Mekusun at sizes that resemble a real model's layers: three periods of [delta memory + dense feed-forward, selective
+    scan + routed experts, latent attention + dense feed-forward, selective scan + routed experts].  A delta memory of
+    width / 64 heads of 64 x 64; a scan over twice the width with 16 state elements per channel, step sizes through a rank of
+    width / 16 and four taps; sixteen attention heads of 128 elements and a rotated part of 64 over a latent of 192; dense
+    feed-forwards of four times the width (no gate: two matrices); 8 experts of twice the width of which 2 are chosen."""
+    mem = {"heads": width // 64, "dim": 64}
+    ssm = {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4}
+    lat = {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 192, "rot_dim": 64, "rot": {"base": 10000.0, "dims": 64}, "scale": (128 + 64) ** -0.5}
+    dense = {"kind": "dense", "ff": 4 * width}
+    moe = {"kind": "moe", "expert": {"ff": 2 * width}, "router": {"experts": 8, "top": 2}}
+    period = [{"type": "general_delta", "mixer": mem, "mlp": dense}, {"type": "mamba1", "mixer": ssm, "mlp": moe},
+              {"type": "latent_attention", "mixer": lat, "mlp": dense}, {"type": "mamba1", "mixer": ssm, "mlp": moe}]
+    return {"architecture": "Mekusun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": float(width) ** 0.5},
+            "logit_softcap": 30.0, "layers": [dict(l) for _ in range(3) for l in period], "max_positions": 4096, "torch_dtype": "bfloat16"}
+
+
+def run_mekusun(dtype: str, context: int, steps: int, warmup: int, widths=(1024, 2048)) -> dict:
+    """Prefill (one prompt of 512 and of 2048 tokens in one step) and decode (1, 8 and 64 requests at ``context``) of
+    Mekusun beside the closest decoders at the same width, twelve layers and vocabulary (random weights): Nesezen (a matrix
+    memory, latent attention, routed experts), Gudutar (a state-space layer with a convolution, latent attention with a
+    rotated part, norms behind the branches) and the Llama decoder."""
+    import torch
+    out = {}
+    for width in widths:
+        models = {
+            "mekusun": mekusun_config(width, 32000),
+            "nesezen": nesezen_config(width, 32000),
+            "gudutar": gudutar_config(width, 3, 32000),
+            "llama": dict(TINYLLAMA, num_hidden_layers=12, hidden_size=width, num_attention_heads=width // 64,
+                          num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
+        }
+        for name, cfg in models.items():
+            row = {}
+            with tempfile.TemporaryDirectory() as folder:
+                engine = make_engine(cfg, folder, dtype, 64, context)
+                for tokens in (512, PREFILL_TOKENS):
+                    t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
+                    row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
+                    row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
+                for batch in (1, 8, 64):
+                    sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
+                    row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
+                    row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
+                row["weights_millions"] = round(sum(_weights_of(engine.model)) / 1e6, 1)
+                del engine
+                torch.cuda.empty_cache()
+            out[f"{name}_w{width}"] = row
+            print(f"[bench] {name} width {width}: {row}", file=sys.stderr, flush=True)
+    return out
+
+
 def _weights_of(model):
     """Numbers of elements of the tensors the model declares (what a checkpoint of it holds)."""
     out = []
@@ -789,7 +841,9 @@ def main() -> int:
                     "matrix memory, latent attention, routed experts with a shared one) beside Gudutar and the Llama decoder at equal width and depth, and nothing else")
     ap.add_argument("--renadra", action="store_true", help="prefill and decode of the Renadra decoder (attention with sigmoid weights beside linear "
                     "attention, windowed attention with normed values, gated recurrences, a bigram embedding, repeated layers) beside Nesezen and the Llama decoder at equal sizes, instead")
-    ap.add_argument("--widths", default=None, metavar="N,N", help="model widths of --renadra (default 1024,2048)")
+    ap.add_argument("--mekusun", action="store_true", help="prefill and decode of the Mekusun decoder (a selective scan, a delta memory, latent attention, "
+                    "ungated experts, a weighted sum over the depth) beside Nesezen, Gudutar and the Llama decoder at equal sizes, instead")
+    ap.add_argument("--widths", default=None, metavar="N,N", help="model widths of --renadra and --mekusun (default 1024,2048)")
     ap.add_argument("--kernels", action="store_true", help="every kernel of a decode step and of a prompt step on its own, with its fraction")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -827,6 +881,12 @@ def main() -> int:
         print(json.dumps({"metric": "Renadra beside Nesezen and the Llama decoder at equal width, layer runs and vocabulary (random weights): prefill and decode",
                           "dtype": short, "context": args.context,
                           "models": run_renadra(args.dtype, args.context, max(16, args.steps // 2), max(4, args.warmup // 2), widths)}))
+        return 0
+    if args.mekusun:
+        widths = tuple(int(w) for w in args.widths.split(",")) if args.widths else (1024, 2048)
+        print(json.dumps({"metric": "Mekusun beside Nesezen, Gudutar and the Llama decoder at equal width, depth and vocabulary (random weights): prefill and decode",
+                          "dtype": short, "context": args.context,
+                          "models": run_mekusun(args.dtype, args.context, max(16, args.steps // 2), max(4, args.warmup // 2), widths)}))
         return 0
     if args.workload == "ragged64":
         print(json.dumps({"metric": f"output tokens/s, 64 ragged requests at once, prompts 64-2048 tokens, 256 generated each ({model_name}, random weights)",

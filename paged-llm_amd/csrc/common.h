@@ -44,6 +44,17 @@ __device__ __forceinline__ float row_activation(float z, int act, float p0 = 0.f
   return act == PLLM_ROW_ACT_TANH ? tanhf(z) : z;
 }
 
+// The same for results that are rounded to bfloat16 next: GELU through the approximation of erf by Abramowitz and Stegun,
+// formula 7.1.26 (absolute error below 1.5e-7), whose complement needs no difference of nearly equal numbers below zero.
+__device__ __forceinline__ float row_activation_for_bf16(float z, int act) {
+  if (act != PLLM_ROW_ACT_GELU) return row_activation(z, act);
+  const float x = fabsf(z) * 0.7071067811865476f;
+  const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, x, 1.f));
+  const float poly = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 1.061405429f, -1.453152027f), 1.421413741f), -0.284496736f), 0.254829592f);
+  const float tail = poly * __builtin_amdgcn_exp2f(-1.4426950408889634f * x * x);      // 1 - erf(x)
+  return 0.5f * z * (z > 0.f ? 2.f - tail : tail);
+}
+
 // Terms of an attention score beside the scaled dot product x = scale * q.k, for mixers that have them:
 //   score(query position i, key position n, head h) = cap(x) + slopes[h] * (n - i),   cap(x) = c tanh(x / c) for c > 0,
 // and a logit sinks[h] that takes part in the softmax's sum and in nothing else (a key with no value).

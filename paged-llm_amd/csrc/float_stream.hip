@@ -852,13 +852,34 @@ __global__ __launch_bounds__(256) void activate_rows_kernel(const TI* in, long i
   out[t * out_stride + c] = from_f32<TO>(row_activation(to_f32(in[t * in_stride + c]), act, p0, p1));
 }
 
+// The same with eight elements per thread and load; cols and both strides multiples of 8, rows on 16-byte boundaries.  blockIdx.y = row.
+template <typename T> struct alignas(16) Eight { T v[8]; };
+
+template <typename TI, typename TO>
+__global__ __launch_bounds__(256) void activate_rows_vec_kernel(const TI* in, long in_stride, TO* out, long out_stride, int cols, int act,
+                                                                float p0, float p1) {
+  const int c = 8 * (blockIdx.x * blockDim.x + threadIdx.x);
+  if (c >= cols) return;
+  const Eight<TI> x = *reinterpret_cast<const Eight<TI>*>(in + (size_t)blockIdx.y * in_stride + c);
+  Eight<TO> y;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) y.v[e] = from_f32<TO>(row_activation(to_f32(x.v[e]), act, p0, p1));
+  *reinterpret_cast<Eight<TO>*>(out + (size_t)blockIdx.y * out_stride + c) = y;
+}
+
 PLLM_API int pllm_activate_rows(int in_dtype, int out_dtype, const void* in, long in_stride, void* out, long out_stride, int num_rows, int cols,
                                 int act, float p0, float p1, hipStream_t stream) {
   if (num_rows <= 0 || cols <= 0) return 0;
   if (act < 0 || act >= PLLM_ROW_ACT_COUNT) return -2;
   const size_t total = (size_t)num_rows * cols;
   dim3 grid((unsigned)((total + 255) / 256)), block(256);
+  const bool vec = cols % 8 == 0 && in_stride % 8 == 0 && out_stride % 8 == 0 && (uintptr_t)in % 16 == 0 && (uintptr_t)out % 16 == 0 && num_rows <= 65535;
+  const int threads = cols >= 2048 ? 256 : (cols / 8 + 63) / 64 * 64;
 #define PLLM_AR(TI, TO)                                                                                                                \
+  if (vec)                                                                                                                             \
+    hipLaunchKernelGGL((activate_rows_vec_kernel<TI, TO>), dim3((cols / 8 + threads - 1) / threads, num_rows), dim3(threads), 0, stream, \
+                       (const TI*)in, in_stride, (TO*)out, out_stride, cols, act, p0, p1);                                             \
+  else                                                                                                                                 \
   hipLaunchKernelGGL((activate_rows_kernel<TI, TO>), grid, block, 0, stream, (const TI*)in, in_stride, (TO*)out, out_stride, cols, act, p0, p1, total)
   if (in_dtype == PLLM_F32) { if (out_dtype == PLLM_F32) PLLM_AR(float, float); else PLLM_AR(float, bf16); }
   else { if (out_dtype == PLLM_F32) PLLM_AR(bf16, float); else PLLM_AR(bf16, bf16); }

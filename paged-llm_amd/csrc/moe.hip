@@ -481,7 +481,7 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
         const float ps = pair_scale ? pair_scale[sorted_pair[row0 + row]] : 1.f;      // a factor on the pair's input row
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          if (col + i < n_out) o[i] = from_f32<bf16>(GATED ? gate_activation(acc[u][0][t][i] * ps, act) * (acc[u][W - 1][t][i] * ps) : row_activation(acc[u][0][t][i] * ps, act));
+          if (col + i < n_out) o[i] = from_f32<bf16>(GATED ? gate_activation(acc[u][0][t][i] * ps, act) * (acc[u][W - 1][t][i] * ps) : row_activation_for_bf16(acc[u][0][t][i] * ps, act));
       } else {
         float* o = reinterpret_cast<float*>(out_) + (size_t)(row0 + row) * ld_out + col;
         if (col + 3 < n_out && (ld_out & 3) == 0) {
@@ -578,7 +578,7 @@ __global__ __launch_bounds__(256) void moe_expert_splitk_kernel(const bf16* __re
     const float ps = pair_scale ? pair_scale[sorted_pair[row0 + r]] : 1.f;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (col + i < n_out) o[i] = from_f32<bf16>(GATED ? gate_activation(acc[0][i] * ps, act) * (acc[W - 1][i] * ps) : row_activation(acc[0][i] * ps, act));
+      if (col + i < n_out) o[i] = from_f32<bf16>(GATED ? gate_activation(acc[0][i] * ps, act) * (acc[W - 1][i] * ps) : row_activation_for_bf16(acc[0][i] * ps, act));
   } else {
     float* o = reinterpret_cast<float*>(out_) + (size_t)(row0 + r) * ld_out + col;
 #pragma unroll
@@ -725,9 +725,16 @@ __global__ __launch_bounds__(256) void moe_expert_tile_kernel(const bf16* __rest
       for (int j = 0; j < 4; ++j) {
         const int col = n0 + wn * 64 + j * 16 + 4 * g;
         bf16* o = reinterpret_cast<bf16*>(out_) + (size_t)(row0 + row) * ld_out + col;
+        struct alignas(8) { bf16 v[4]; } y;
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (col + i < n_out) o[i] = from_f32<bf16>(row_activation(acc[j][t][i] * ps, act));
+        for (int i = 0; i < 4; ++i) y.v[i] = from_f32<bf16>(row_activation_for_bf16(acc[j][t][i] * ps, act));
+        if (col + 3 < n_out && (ld_out & 3) == 0) {
+          *reinterpret_cast<decltype(y)*>(o) = y;
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (col + i < n_out) o[i] = y.v[i];
+        }
       }
     } else {
 #pragma unroll

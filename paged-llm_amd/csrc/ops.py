@@ -1505,6 +1505,9 @@ def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor,
 
 
 DELTA_MAX_DIM = 256               # size of a head that the delta memory takes
+DELTA_CHUNK = 32                  # tokens that its kernels for long portions work off as matrices
+DELTA_CHUNK_MAX_DIM = 128         # ... for heads up to this size
+DELTA_CHUNKS_FROM = 48            # tokens of the longest sequence of a step from which those kernels run
 
 
 def delta_rule(rows: torch.Tensor, columns: dict, raw_w: torch.Tensor, w0: torch.Tensor, bias_a: torch.Tensor, weight: torch.Tensor, eps: float,
@@ -1515,7 +1518,9 @@ def delta_rule(rows: torch.Tensor, columns: dict, raw_w: torch.Tensor, w0: torch
     weight * sigmoid(gate).  ``rows`` [T, ...] holds r, k, v, raw_a and the gate, heads * dim columns each, from the columns
     ``columns`` = {"r", "k", "v", "a", "g"} on (unit inner stride); raw_w float32 [T, heads * dim]; w0, bias_a, weight float32
     [heads * dim].  S float32 [heads, dim, dim] in front of ``state[slot]``; a sequence with seq_starts == 0 starts from
-    S = 0.  Returns [T, heads * dim] in the rows' type."""
+    S = 0.  Returns [T, heads * dim] in the rows' type.  From ``DELTA_CHUNKS_FROM`` tokens of one sequence on (``max_q_len``) the
+    sequences are worked off in chunks of ``DELTA_CHUNK`` tokens as matrix products in float, which round differently than
+    token by token."""
     _on_gpu(rows, raw_w, w0, bias_a, weight, state, state_slots, seq_starts, cu_seqlens)
     T, C = rows.shape[0], heads * dim
     _need(rows.dim() == 2 and rows.stride(1) == 1 and all(0 <= columns[n] and columns[n] + C <= rows.shape[1] for n in "rkvag"),
@@ -1526,6 +1531,18 @@ def delta_rule(rows: torch.Tensor, columns: dict, raw_w: torch.Tensor, w0: torch
         _need(t.dtype == torch.float32 and t.shape == (C,) and t.is_contiguous(), f"{what}: float32 [{C}]")
     _check_sequences(state, state_slots, seq_starts, cu_seqlens, num_seqs)
     _need(heads * dim * dim <= state.shape[1], "the memory does not fit the state slot")
+    if max_q_len >= DELTA_CHUNKS_FROM and dim <= DELTA_CHUNK_MAX_DIM:
+        max_chunks = T // DELTA_CHUNK + num_seqs
+        per_chunk = _fn("delta_rule.hip", "pllm_delta_chunk_floats", signature=[c_int, c_int])(heads, dim)
+        ws = torch.empty(max_chunks * per_chunk, dtype=torch.float32, device=rows.device)
+        y = torch.empty((T, C), dtype=torch.float32, device=rows.device)
+        sig = [c_int, c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p,
+               c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p]
+        _check(_fn("delta_rule.hip", "pllm_delta_rule_chunks", signature=sig)(
+            dtype_code(rows.dtype), _ptr(rows), rows.stride(0), columns["r"], columns["k"], columns["v"], columns["a"], _ptr(raw_w), raw_w.stride(0),
+            _ptr(w0), _ptr(bias_a), _ptr(state), state.stride(0), _ptr(state_slots), _ptr(seq_starts), _ptr(cu_seqlens), _ptr(y), num_seqs, heads,
+            dim, max_chunks, _ptr(ws), _stream()), "delta_rule_chunks")
+        return gated_group_norm(y, rows[:, columns["g"]:columns["g"] + C], weight, dim, False, eps, gate_activation="sigmoid")
     out = torch.empty((T, C), dtype=rows.dtype, device=rows.device)
     sig = [c_int, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_float, c_void_p,
            c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]

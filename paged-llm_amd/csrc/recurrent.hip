@@ -629,6 +629,48 @@ __global__ __launch_bounds__(256) void gated_group_norm_regs_kernel(const float*
   }
 }
 
+// The same for small groups, whose lanes (four channels each, a power of two of them, at most 32) lie side by side in a
+// wavefront: every lane works, where the kernel above would leave most of a wavefront without channels.
+template <typename T>
+__global__ __launch_bounds__(256) void gated_group_norm_lanes_kernel(const float* __restrict__ y, const T* __restrict__ gate,
+                                                                     int gate_stride, const float* __restrict__ w, T* __restrict__ out,
+                                                                     int inner, int group, int gate_first, int gate_act, float eps) {
+  const int row = blockIdx.y, at = 4 * (blockIdx.x * blockDim.x + threadIdx.x), lanes = group / 4;
+  const bool in = at < inner;                                // (inner is a multiple of the group: a group is in or out as a whole)
+  float u[4] = {0.f, 0.f, 0.f, 0.f}, s[4] = {1.f, 1.f, 1.f, 1.f};
+  float ss = 0.f;
+  if (in) {
+    const float4 yv = *reinterpret_cast<const float4*>(y + (size_t)row * inner + at);
+    u[0] = yv.x; u[1] = yv.y; u[2] = yv.z; u[3] = yv.w;
+    if (gate_act != kGateNone) {
+      const Quad<T> gv = *reinterpret_cast<const Quad<T>*>(gate + (size_t)row * gate_stride + at);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s[e] = gate_f32(to_f32(gv.v[e]), gate_act);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (gate_first) u[e] *= s[e];
+      ss = fmaf(u[e], u[e], ss);
+    }
+  }
+  for (int off = 1; off < lanes; off <<= 1) ss += __shfl_xor(ss, off, 64);
+  if (!in) return;
+  const float inv = 1.f / sqrtf(ss / (float)group + eps);
+  Quad<T> o;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    float r = gate_first ? u[e] * inv : (u[e] * inv) * s[e];
+    if (w) r *= w[at + e];
+    o.v[e] = from_f32<T>(r);
+  }
+  *reinterpret_cast<Quad<T>*>(out + (size_t)row * inner + at) = o;
+}
+
+static bool group_norm_in_lanes(int inner, int group, int num_tokens) {
+  const int lanes = group / 4;
+  return group <= 128 && (lanes & (lanes - 1)) == 0 && inner / group >= 4 && num_tokens <= 65535;
+}
+
 template <typename T>
 static bool group_norm_in_registers(const float* y, const void* gate, int gate_stride, void* out, int inner, int group) {
   const int groups = inner / group, parts = groups >= 4 ? 1 : 4 / groups;
@@ -641,15 +683,23 @@ PLLM_API int pllm_gated_group_norm(int dtype, const float* y, const void* gate, 
   if (num_tokens <= 0) return 0;
   if (group <= 0 || inner % group || gate_act < 0 || gate_act > kGateNone || (!gate && gate_act != kGateNone)) return -2;
   dim3 grid(num_tokens), block(256);
+  const int quads = (inner + 3) / 4;
+  dim3 lanes_block(quads >= 256 ? 256 : (quads + 63) / 64 * 64), lanes_grid((quads + lanes_block.x - 1) / lanes_block.x, num_tokens);
   if (dtype == PLLM_F32) {
-    if (group_norm_in_registers<float>(y, gate, gate_stride, out, inner, group))
+    if (group_norm_in_registers<float>(y, gate, gate_stride, out, inner, group) && group_norm_in_lanes(inner, group, num_tokens))
+      hipLaunchKernelGGL(gated_group_norm_lanes_kernel<float>, lanes_grid, lanes_block, 0, stream, y, (const float*)gate, gate_stride, w, (float*)out,
+                         inner, group, gate_first, gate_act, eps);
+    else if (group_norm_in_registers<float>(y, gate, gate_stride, out, inner, group))
       hipLaunchKernelGGL(gated_group_norm_regs_kernel<float>, grid, block, 0, stream, y, (const float*)gate, gate_stride, w, (float*)out,
                          inner, group, gate_first, gate_act, eps);
     else
       hipLaunchKernelGGL(gated_group_norm_kernel<float>, grid, block, 0, stream, y, (const float*)gate, gate_stride, w, (float*)out,
                          inner, group, gate_first, gate_act, eps);
   } else {
-    if (group_norm_in_registers<bf16>(y, gate, gate_stride, out, inner, group))
+    if (group_norm_in_registers<bf16>(y, gate, gate_stride, out, inner, group) && group_norm_in_lanes(inner, group, num_tokens))
+      hipLaunchKernelGGL(gated_group_norm_lanes_kernel<bf16>, lanes_grid, lanes_block, 0, stream, y, (const bf16*)gate, gate_stride, w, (bf16*)out,
+                         inner, group, gate_first, gate_act, eps);
+    else if (group_norm_in_registers<bf16>(y, gate, gate_stride, out, inner, group))
       hipLaunchKernelGGL(gated_group_norm_regs_kernel<bf16>, grid, block, 0, stream, y, (const bf16*)gate, gate_stride, w, (bf16*)out,
                          inner, group, gate_first, gate_act, eps);
     else
