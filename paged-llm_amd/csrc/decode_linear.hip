@@ -5,7 +5,7 @@
 //                         residual is written out by workgroup 0; RMS norm in float: the elements
 //                         take the norm's weights here, the row's 1 / rms goes onto the finished sums
 //   product               rows[M, K] * W[N, K]^T on the matrix cores, float accumulation
-//   epilogue              plain (bfloat16 or float out) | act(gate) * up | rotary encoding of q and
+//   epilogue              plain (bfloat16 or float out) | act(row) | act(gate) * up | rotary encoding of q and
 //                         k and the write of k, v into their cache pages
 //
 // One workgroup of 8 wavefronts owns units of 16 weight rows over all of K.  Its wavefronts deal the K
@@ -27,7 +27,7 @@ constexpr int kSlab = 128;
 constexpr int kPad = 8;            // bf16 elements of padding per LDS row (spreads rows over banks)
 constexpr int kSquares = 512;      // floats of LDS for the rows' sums of squares: 16 rows x up to 32 column groups of 512
 
-enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_GATED = 2, EPI_ROPE_KV = 3 };
+enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_GATED = 2, EPI_ROPE_KV = 3, EPI_ACT = 4 };
 
 struct DecodeLinearParams {
   const bf16* x; int ldx;
@@ -44,6 +44,7 @@ struct DecodeLinearParams {
   const int* positions; const float* cos_t; const float* sin_t; const int* slots;
   bf16* k_pages; bf16* v_pages;
   int num_heads, num_kv_heads, head_dim, block_size;
+  float act_p0, act_p1;        // EPI_ACT: the activation's parameters (`activation` is one of PLLM_ROW_ACT_* then)
 };
 
 __device__ __forceinline__ bf16x8 zero8() {
@@ -388,12 +389,12 @@ __global__ __launch_bounds__(WAVES * 64) void decode_linear_kernel(const DecodeL
       if (HALF) {
         // useful blocks: (rows 0-7, columns 0-7) + (rows 8-15, columns 8-15), 40 lanes further
         if (m < M && m < 8 && row < 8) {
-          if (EPI == EPI_BF16 || EPI == EPI_F32) {
+          if (EPI == EPI_BF16 || EPI == EPI_F32 || EPI == EPI_ACT) {
             const int n = unit * 8 + row;
             if (n < N) {
               const float v = (total(lane) + total(lane + 40)) * row_scale;
               if (EPI == EPI_F32) ((float*)p.out)[(size_t)m * p.ldo + n] = v;
-              else ((bf16*)p.out)[(size_t)m * p.ldo + n] = __float2bfloat16(v);
+              else ((bf16*)p.out)[(size_t)m * p.ldo + n] = __float2bfloat16(EPI == EPI_ACT ? row_activation(v, p.activation, p.act_p0, p.act_p1) : v);
             }
           } else if (EPI == EPI_ROPE_KV && row < 4) {
             const int d = p.head_dim, half = d >> 1, per_head = half >> 2;
@@ -403,12 +404,12 @@ __global__ __launch_bounds__(WAVES * 64) void decode_linear_kernel(const DecodeL
           }
         }
       } else if (m < M) {
-        if (EPI == EPI_BF16 || EPI == EPI_F32) {
+        if (EPI == EPI_BF16 || EPI == EPI_F32 || EPI == EPI_ACT) {
           const int n = unit * 16 + row;
           if (n < N) {
             const float v = total(lane) * row_scale;
             if (EPI == EPI_F32) ((float*)p.out)[(size_t)m * p.ldo + n] = v;
-            else ((bf16*)p.out)[(size_t)m * p.ldo + n] = __float2bfloat16(v);
+            else ((bf16*)p.out)[(size_t)m * p.ldo + n] = __float2bfloat16(EPI == EPI_ACT ? row_activation(v, p.activation, p.act_p0, p.act_p1) : v);
           }
         } else if (EPI == EPI_GATED) {
           const int n = unit * 8 + row;
@@ -562,12 +563,12 @@ __global__ __launch_bounds__(512) void decode_linear_wide_kernel(const DecodeLin
         };
         const int m = row0 + t * 16 + r;
         if (m >= M) continue;
-        if (EPI == EPI_BF16 || EPI == EPI_F32) {
+        if (EPI == EPI_BF16 || EPI == EPI_F32 || EPI == EPI_ACT) {
           const int n = unit * 16 + row;
           if (n < N) {
             const float v = total(lane);
             if (EPI == EPI_F32) ((float*)p.out)[(size_t)m * p.ldo + n] = v;
-            else ((bf16*)p.out)[(size_t)m * p.ldo + n] = __float2bfloat16(v);
+            else ((bf16*)p.out)[(size_t)m * p.ldo + n] = __float2bfloat16(EPI == EPI_ACT ? row_activation(v, p.activation, p.act_p0, p.act_p1) : v);
           }
         } else if (EPI == EPI_GATED) {
           const int n = unit * 8 + row;
@@ -675,9 +676,9 @@ PLLM_API int pllm_decode_linear(int epi, const void* x, int ldx, const void* del
                                 void* x_out, int ldxo, const int* row_index, const void* W, int ldw, const void* Wt, void* out, int ldo, int M,
                                 int N, int K, const int* positions, const float* cos_t, const float* sin_t, const int* slots,
                                 void* k_pages, void* v_pages, int num_heads, int num_kv_heads, int head_dim, int block_size,
-                                int activation, hipStream_t stream) {
+                                int activation, float act_p0, float act_p1, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
-  if (activation < 0 || activation >= PLLM_ACT_COUNT) return -2;
+  if (activation < 0 || activation >= (epi == EPI_ACT ? PLLM_ROW_ACT_COUNT : PLLM_ACT_COUNT)) return -2;
   if (M > 64 || (M > 16 && (delta || norm_w)) || K <= 0 || (K & 7) || (ldx & 7) || (W && (ldw & 7)) || (delta && (ldd & 7)) || (x_out && (ldxo & 7))) return -2;
   if ((!W && !Wt) || (Wt && (K & 31)) || (!W && M > 16)) return -2;
   DecodeLinearParams p;
@@ -685,10 +686,10 @@ PLLM_API int pllm_decode_linear(int epi, const void* x, int ldx, const void* del
   p.x_out = (bf16*)x_out; p.ldxo = ldxo; p.row_index = row_index; p.W = (const bf16*)W; p.ldw = ldw; p.Wt = (const bf16*)Wt; p.out = out; p.ldo = ldo;
   p.M = M; p.N = N; p.K = K; p.positions = positions; p.cos_t = cos_t; p.sin_t = sin_t; p.slots = slots;
   p.k_pages = (bf16*)k_pages; p.v_pages = (bf16*)v_pages; p.num_heads = num_heads; p.num_kv_heads = num_kv_heads;
-  p.head_dim = head_dim; p.block_size = block_size; p.activation = activation;
+  p.head_dim = head_dim; p.block_size = block_size; p.activation = activation; p.act_p0 = act_p0; p.act_p1 = act_p1;
   int units;
   switch (epi) {
-    case EPI_BF16: case EPI_F32: units = (N + 15) / 16; break;
+    case EPI_BF16: case EPI_F32: case EPI_ACT: units = (N + 15) / 16; break;
     case EPI_GATED: units = (N + 7) / 8; break;
     case EPI_ROPE_KV:
       if (head_dim % 16 || !slots || !k_pages || !v_pages || N != (num_heads + 2 * num_kv_heads) * head_dim) return -2;
@@ -709,6 +710,7 @@ PLLM_API int pllm_decode_linear(int epi, const void* x, int ldx, const void* del
     switch (epi) {
       case EPI_BF16: return launch_wide<EPI_BF16>(p, units, blocks, cus, stream);
       case EPI_F32: return launch_wide<EPI_F32>(p, units, blocks, cus, stream);
+      case EPI_ACT: return launch_wide<EPI_ACT>(p, units, blocks, cus, stream);
       case EPI_GATED: return launch_wide<EPI_GATED>(p, units, blocks, cus, stream);
       case EPI_ROPE_KV: return launch_wide<EPI_ROPE_KV>(p, units, blocks, cus, stream);
     }
@@ -746,12 +748,14 @@ PLLM_API int pllm_decode_linear(int epi, const void* x, int ldx, const void* del
     switch (epi) {
       case EPI_BF16: GO(EPI_BF16, true);
       case EPI_F32: GO(EPI_F32, true);
+      case EPI_ACT: GO(EPI_ACT, true);
       case EPI_ROPE_KV: GO(EPI_ROPE_KV, true);
     }
   }
   switch (epi) {
     case EPI_BF16: GO(EPI_BF16, false);
     case EPI_F32: GO(EPI_F32, false);
+    case EPI_ACT: GO(EPI_ACT, false);
     case EPI_GATED: GO(EPI_GATED, false);
     case EPI_ROPE_KV: GO(EPI_ROPE_KV, false);
   }

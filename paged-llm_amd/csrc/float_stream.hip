@@ -384,7 +384,7 @@ __global__ __launch_bounds__(kHeldThreads) void rms_sandwich_held_kernel(const f
 struct DepthSum {
   float* history; long plane; const float* weights; int count;
 };
-constexpr int kDepthAhead = 4;            // planes whose rows are asked for at once
+constexpr int kDepthAhead = 8;            // planes whose rows are asked for at once
 
 template <typename TO, typename TH, int VEC>
 __global__ __launch_bounds__(kHeldThreads) void rms_depth_kernel(const float* __restrict__ branch, const ChoiceSum sum, const DepthSum depth,

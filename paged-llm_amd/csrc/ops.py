@@ -466,12 +466,12 @@ def sample(logits: torch.Tensor, temperature: torch.Tensor, top_k: torch.Tensor,
 
 
 # ------------------------------------------------------------------------------------------- fused decode products
-EPI_BF16, EPI_F32, EPI_GATED, EPI_ROPE_KV = 0, 1, 2, 3
+EPI_BF16, EPI_F32, EPI_GATED, EPI_ROPE_KV, EPI_ACT = 0, 1, 2, 3, 4
 DECODE_MAX_ROWS = 16          # rows of the fused form with a sum or norm in front
 DECODE_WIDE_MAX_ROWS = 64     # rows of the form for plain rows
 _DECODE_SIG = [c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-               c_int, c_void_p]
+               c_int, c_float, c_float, c_void_p]
 _lds_limit: dict = {}
 
 
@@ -526,12 +526,12 @@ def decode_linear_pays(rows: int, N: int, K: int, epi: int, staged: bool) -> boo
 def decode_linear(x: torch.Tensor, w: torch.Tensor, epi: int = EPI_BF16, delta: torch.Tensor | None = None,
                   norm_weight: torch.Tensor | None = None, eps: float = 0.0, x_out: torch.Tensor | None = None,
                   row_index: torch.Tensor | None = None, rope: dict | None = None, tiled=None,
-                  activation: str = "silu") -> torch.Tensor:
+                  activation: str = "silu", act_params: tuple = (0.0, 0.0)) -> torch.Tensor:
     """rows = x[row_index] (+ delta) -> optional RMS norm -> rows W^T -> epilogue, in one kernel.
     ``tiled``: the matrix's ``TiledWeight`` with the pairing that goes with ``epi`` (at most 16 rows): the weights are then
     streamed from that copy, in contiguous pieces, wherever the kernel works in units of 16 weight rows.
 
-    epi EPI_BF16 / EPI_F32: [M, N] out.  EPI_GATED: w = [gate; up], out = act(gate) * up [M, N/2] (``activation``).
+    epi EPI_BF16 / EPI_F32: [M, N] out.  EPI_ACT: act(out) [M, N] (``activation`` one of ``ROW_ACTIVATIONS`` with ``act_params``).  EPI_GATED: w = [gate; up], out = act(gate) * up [M, N/2] (``activation``).
     EPI_ROPE_KV: w = [q; k; v] rows; q is rotated and returned [M, heads * d]; k (rotated) and v go
     into the cache pages; ``rope`` = dict(positions, cos, sin, slots, k_pages, v_pages, num_heads,
     num_kv_heads, head_dim, block_size).  ``x_out`` receives x + delta (the new residual).
@@ -586,15 +586,16 @@ def decode_linear(x: torch.Tensor, w: torch.Tensor, epi: int = EPI_BF16, delta: 
              None if tiled is None else _ptr(tiled.tiles), _ptr(out),
              out.stride(0), M, N, K, _ptr(r.get("positions")), _ptr(r.get("cos")), _ptr(r.get("sin")), _ptr(r.get("slots")),
              _ptr(r.get("k_pages")), _ptr(r.get("v_pages")), int(r.get("num_heads", 0)), int(r.get("num_kv_heads", 0)),
-             int(r.get("head_dim", 0)), int(r.get("block_size", 0)), activation_code(activation), _stream()), "decode_linear")
+             int(r.get("head_dim", 0)), int(r.get("block_size", 0)), row_activation_code(activation) if epi == EPI_ACT else activation_code(activation),
+             c_float(act_params[0]), c_float(act_params[1]), _stream()), "decode_linear")
     return out
 
 
 # ------------------------------------------------------------------------------------------- products of 17 to a few hundred rows
-SL_BF16, SL_F32, SL_GATED, SL_PARTIAL, SL_ROPE_KV = 0, 1, 2, 3, 4
+SL_BF16, SL_F32, SL_GATED, SL_PARTIAL, SL_ROPE_KV, SL_ACT = 0, 1, 2, 3, 4, 5
 STREAM_TILE_ROWS, STREAM_TILE_K = 16, 32
 _STREAM_SIG = [c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p,
-               c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p]
+               c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p]
 
 
 class TiledWeight:
@@ -681,8 +682,8 @@ def gated_blocks_per_workgroup(out_features: int, compute_units: int) -> int:
 
 
 def stream_linear(x: torch.Tensor, w: TiledWeight, epi: int = SL_BF16, nt: int | None = None, splits: int | None = None,
-                  rope: dict | None = None, activation: str = "silu") -> torch.Tensor:
-    """x [M, K] bfloat16 times the tiled weights.  SL_BF16 / SL_F32: [M, N]; SL_GATED: act(gate) * up [M, N / 2];
+                  rope: dict | None = None, activation: str = "silu", act_params: tuple = (0.0, 0.0)) -> torch.Tensor:
+    """x [M, K] bfloat16 times the tiled weights.  SL_BF16 / SL_F32: [M, N]; SL_ACT: act of it (one of ``ROW_ACTIVATIONS`` with ``act_params``); SL_GATED: act(gate) * up [M, N / 2];
     SL_PARTIAL: float [splits, M, N], the sums over ``splits`` ranges of K, to be added in that order; SL_ROPE_KV: q rotated
     [M, heads * d], k (rotated) and v written to their pages (``rope`` as for ``decode_linear``)."""
     _on_gpu(x, w.tiles)
@@ -725,7 +726,8 @@ def stream_linear(x: torch.Tensor, w: TiledWeight, epi: int = SL_BF16, nt: int |
     _check(f(epi, _ptr(x), x.stride(0), _ptr(w.tiles), _ptr(out), out.stride(-2), M, N, K, w.blocks, nt, splits,
              _ptr(r.get("positions")), _ptr(r.get("cos")), _ptr(r.get("sin")), _ptr(r.get("slots")), _ptr(r.get("k_pages")),
              _ptr(r.get("v_pages")), int(r.get("num_heads", 0)), int(r.get("num_kv_heads", 0)), int(r.get("head_dim", 0)),
-             int(r.get("block_size", 0)), activation_code(activation), _stream()), "stream_linear")
+             int(r.get("block_size", 0)), row_activation_code(activation) if epi == SL_ACT else activation_code(activation),
+             c_float(act_params[0]), c_float(act_params[1]), _stream()), "stream_linear")
     return out
 
 
@@ -1473,7 +1475,7 @@ def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor,
                    num_seqs: int, max_q_len: int = 0) -> torch.Tensor:
     """S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,  y_c = sum_n S[c, n] C_n + skip_c x_c,  out = y silu(z), with
     dt = softplus(raw_dt + dt_bias).  x, z [T, channels] (views of one type, unit inner stride), raw_dt contiguous float32
-    [T, channels], bc float32 [T, 2 N] (a view: B, then C), a2 float32 [N, channels] = A log2(e) transposed, N as
+    [T, channels], bc [T, 2 N] of x's type (a view: B, then C; rows on 4-byte boundaries), a2 float32 [N, channels] = A log2(e) transposed, N as
     ``scan_state_size`` gives it; S float32 [N, channels] in front of ``state[slot]``; a sequence with seq_starts == 0 starts
     from S = 0.  Returns [T, channels] in x's type.  From ``SCAN_CHUNKS_FROM`` tokens of one sequence on (``max_q_len``) the
     sequences run in chunks side by side, which rounds differently than token by token."""
@@ -1483,7 +1485,8 @@ def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor,
     _need(x.stride(1) == 1 and z.shape == (T, C) and z.stride(1) == 1 and z.dtype == x.dtype, "selective_scan x, z: [T, channels] of one type, unit inner stride")
     _need(raw_dt.dtype == torch.float32 and raw_dt.shape == (T, C) and raw_dt.is_contiguous(), f"raw_dt: contiguous float32 [{T}, {C}]")
     _need(scan_state_size(N) == N and N <= SCAN_STATE_MAX, f"a state of {N} per channel: 8, 16 or a multiple of 32 up to {SCAN_STATE_MAX}")
-    _need(bc.dtype == torch.float32 and bc.shape == (T, 2 * N) and bc.stride(1) == 1, f"bc: float32 [{T}, {2 * N}] with unit inner stride")
+    _need(bc.dtype == x.dtype and bc.shape == (T, 2 * N) and bc.stride(1) == 1 and bc.data_ptr() % 4 == 0 and bc.stride(0) * bc.element_size() % 4 == 0,
+          f"bc: [{T}, {2 * N}] of x's type with unit inner stride, rows on 4-byte boundaries")
     _need(a2.dtype == torch.float32 and a2.shape == (N, C) and a2.is_contiguous(), f"a2: float32 [{N}, {C}]")
     for t, what in ((dt_bias, "dt_bias"), (skip, "skip")):
         _need(t.dtype == torch.float32 and t.shape == (C,) and t.is_contiguous(), f"{what}: float32 [{C}]")
@@ -1495,6 +1498,8 @@ def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor,
     ws_state = torch.empty((max_chunks, N * C), dtype=torch.float32, device=x.device) if chunk else None
     ws_steps = torch.empty((max_chunks, C), dtype=torch.float32, device=x.device) if chunk else None
     dt = torch.empty((T, C), dtype=torch.float32, device=x.device) if chunk else None
+    if chunk and bc.dtype != torch.float32:
+        bc = activate_rows(bc, None, out_dtype=torch.float32)          # (the same numbers: the passes over chunks read them as float)
     sig = [c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_long,
            c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p]
     _check(_fn("selective_scan.hip", "pllm_selective_scan", signature=sig)(

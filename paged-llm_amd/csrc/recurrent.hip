@@ -30,7 +30,8 @@ __device__ __forceinline__ float gate_f32(float z, int act) { return act == kGat
 
 // ---------------------------------------------------------------------------------------------
 constexpr int kMaxTaps = 16;      // most taps of a filter; filters of up to 8 taps take the smaller instance of the kernels
-constexpr int kConvChunk = 64;     // tokens of one sequence that one workgroup walks
+constexpr int kConvChunk = 64;     // tokens of one sequence that one workgroup walks: up to so many in one go (its state is then left by
+constexpr int kConvShort = 16;     // the same kernel), else so many at a time, for workgroups enough to fill the GPU
 
 // out[t, c] = act(bias[c] + sum_j w[c, j] * in[t - (taps - 1) + j, c]); the last column of w meets the current token;
 // inputs before the sequence's first token of this step come from the state (or are zero for a sequence that starts).
@@ -40,13 +41,13 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
     const T* __restrict__ in, int in_stride, const float* __restrict__ w, const float* __restrict__ bias,
     float* state, size_t slot_stride, const int* __restrict__ state_slots,
     const int* __restrict__ seq_starts, const int* __restrict__ cu_seqlens, T* __restrict__ out, int out_stride,
-    int channels, int taps, int act, int leave_state) {
+    int channels, int taps, int act, int leave_state, int chunk) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   const int seq = blockIdx.y;
   const int q_begin = cu_seqlens[seq], q_len = cu_seqlens[seq + 1] - q_begin;
-  const int t0 = blockIdx.z * kConvChunk;
+  const int t0 = blockIdx.z * chunk;
   if (c >= channels || t0 >= q_len) return;
-  const int t1 = t0 + kConvChunk < q_len ? t0 + kConvChunk : q_len;
+  const int t1 = t0 + chunk < q_len ? t0 + chunk : q_len;
   const bool carried = seq_starts[seq] > 0;
   float* st = state + (size_t)state_slots[seq] * slot_stride + (size_t)c * (taps - 1);
   float wj[MAXT], win[MAXT];
@@ -127,11 +128,12 @@ template <typename T, int MAXT>
 static void launch_causal_conv(const void* in, int in_stride, const float* w, const float* bias, float* state, long slot_stride,
                                const int* state_slots, const int* seq_starts, const int* cu_seqlens, void* out, int out_stride,
                                int channels, int taps, int act, int num_seqs, int max_q_len, hipStream_t stream) {
-  dim3 block(256), grid((channels + 255) / 256, num_seqs, (max_q_len + kConvChunk - 1) / kConvChunk);
+  const int chunk = max_q_len <= kConvChunk ? kConvChunk : kConvShort;
+  dim3 block(256), grid((channels + 255) / 256, num_seqs, (max_q_len + chunk - 1) / chunk);
   dim3 grid_state((channels + 255) / 256, num_seqs);
   const int fused = grid.z == 1 && taps > 1;
   hipLaunchKernelGGL((causal_conv_kernel<T, MAXT>), grid, block, 0, stream, (const T*)in, in_stride, w, bias, state,
-                     (size_t)slot_stride, state_slots, seq_starts, cu_seqlens, (T*)out, out_stride, channels, taps, act, fused);
+                     (size_t)slot_stride, state_slots, seq_starts, cu_seqlens, (T*)out, out_stride, channels, taps, act, fused, chunk);
   if (taps > 1 && !fused)
     hipLaunchKernelGGL((conv_state_update_kernel<T, MAXT>), grid_state, block, 0, stream, (const T*)in, in_stride, state,
                        (size_t)slot_stride, state_slots, seq_starts, cu_seqlens, channels, taps);

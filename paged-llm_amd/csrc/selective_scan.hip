@@ -7,7 +7,8 @@
 // the slot held.  All arithmetic is float; T is the storage type of x, z and the output rows.
 //
 // One lane per channel with its states in registers.  B and C of a token are the same numbers for every channel, so a
-// wavefront reads them through the scalar path (float rows [T, 2 N]).  N is 8, 16 or a multiple of 32: a caller with another
+// wavefront reads them through the scalar path (rows [T, 2 N] of type T, in the passes over chunks float: there taking pairs of
+// bfloat16 elements apart would cost more than it saves).  N is 8, 16 or a multiple of 32: a caller with another
 // size pads A, B and C with zeros, and the padded states stay zero.  States of more than 32 elements are cut over the
 // workgroup's wavefronts, whose partial outputs meet in LDS.  A is held as A log2(e), so that a decay is one multiply and one
 // hardware exponential.
@@ -41,6 +42,13 @@ __device__ __forceinline__ float softplus_f32(float z) {
   return fmaxf(z, 0.f) + l;
 }
 
+// Element i of a row that the whole wavefront reads: bfloat16 elements come in pairs (the scalar path has no loads of 16 bits).
+__device__ __forceinline__ float uniform_element(const float* row, int i) { return row[i]; }
+__device__ __forceinline__ float uniform_element(const bf16* row, int i) {
+  const uint32_t pair = reinterpret_cast<const uint32_t*>(row)[i >> 1];
+  return __uint_as_float((i & 1) ? pair & 0xffff0000u : pair << 16);
+}
+
 enum { kScanWhole = 0, kScanState = 1, kScanOut = 2 };
 constexpr int kScanAhead = 4;            // tokens whose rows are asked for at once
 
@@ -58,8 +66,8 @@ __device__ __forceinline__ bool scan_chunk_of(const int* __restrict__ cu, int nu
 // contribution from a zero state, walked from its last token to its first (the decays behind a token are then one
 // exponential of A times the step sizes summed so far), and the softplus of its step sizes.  kScanOut: a chunk's tokens
 // from the state the sequence had when the chunk began.
-template <typename T, int NR, int MAX_THREADS, int MODE>
-__global__ __launch_bounds__(MAX_THREADS) void selective_scan_kernel(ScanArgs a, const float* __restrict__ bc, long bc_stride) {
+template <typename T, typename TB, int NR, int MAX_THREADS, int MODE>
+__global__ __launch_bounds__(MAX_THREADS) void selective_scan_kernel(ScanArgs a, const TB* __restrict__ bc, long bc_stride) {
   __shared__ float part[2][MAX_THREADS / 64][64];
   const int lane = threadIdx.x & 63, wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), waves = blockDim.x >> 6;
   int seq = blockIdx.y, local = 0;
@@ -104,22 +112,22 @@ __global__ __launch_bounds__(MAX_THREADS) void selective_scan_kernel(ScanArgs a,
       if (tb + u >= t_last) break;
       const int t = MODE == kScanState ? t_last - 1 - (tb + u - t_first) : tb + u;
       const float x = to_f32(xv[u]);
-      const float* row = bc + (size_t)(q_begin + t) * bc_stride;       // B, then C
+      const TB* row = bc + (size_t)(q_begin + t) * bc_stride;           // B, then C
       float dt = rv[u];
       if (MODE != kScanOut) dt = softplus_f32(dt + bias);     // (kScanOut: the first pass has left it)
       const float dx = dt * x;
       if (MODE == kScanState) {
         if (ok && wv == 0) dp[(size_t)t * C] = dt;
 #pragma unroll
-        for (int i = 0; i < NR; ++i) S[i] = fmaf(__builtin_amdgcn_exp2f(A[i] * behind), dx * row[n0 + i], S[i]);
+        for (int i = 0; i < NR; ++i) S[i] = fmaf(__builtin_amdgcn_exp2f(A[i] * behind), dx * uniform_element(row, n0 + i), S[i]);
         behind += dt;
         continue;
       }
       float y[2] = {0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < NR; ++i) {
-        S[i] = fmaf(__builtin_amdgcn_exp2f(A[i] * dt), S[i], dx * row[n0 + i]);
-        y[i & 1] = fmaf(S[i], row[a.N + n0 + i], y[i & 1]);
+        S[i] = fmaf(__builtin_amdgcn_exp2f(A[i] * dt), S[i], dx * uniform_element(row, n0 + i));
+        y[i & 1] = fmaf(S[i], uniform_element(row, a.N + n0 + i), y[i & 1]);
       }
       float total = y[0] + y[1];
       if (waves > 1) {
@@ -177,11 +185,11 @@ __global__ __launch_bounds__(256) void selective_scan_carry_kernel(ScanArgs a) {
   *slot = S;
 }
 
-template <typename T, int MODE>
-static void launch_scan(const ScanArgs& a, const float* bc, long bc_stride, int rows, hipStream_t stream) {
+template <typename T, typename TB, int MODE>
+static void launch_scan(const ScanArgs& a, const void* bc, long bc_stride, int rows, hipStream_t stream) {
   const int waves = (a.N + 31) / 32;
   dim3 grid((a.channels + 63) / 64, rows), block(64 * waves);
-#define PLLM_SCAN(NR, MAX_THREADS) hipLaunchKernelGGL((selective_scan_kernel<T, NR, MAX_THREADS, MODE>), grid, block, 0, stream, a, bc, bc_stride)
+#define PLLM_SCAN(NR, MAX_THREADS) hipLaunchKernelGGL((selective_scan_kernel<T, TB, NR, MAX_THREADS, MODE>), grid, block, 0, stream, a, (const TB*)bc, bc_stride)
   if (a.N == 8) PLLM_SCAN(8, 256);
   else if (a.N == 16) PLLM_SCAN(16, 256);
   else if (waves <= 4) PLLM_SCAN(32, 256);
@@ -189,10 +197,10 @@ static void launch_scan(const ScanArgs& a, const float* bc, long bc_stride, int 
 #undef PLLM_SCAN
 }
 
-// chunk == 0: every sequence token by token.  chunk > 0: three passes over chunks of that many tokens; ws_state holds
+// bc: [T, 2 N] of type dtype, or (chunk > 0) float.  chunk == 0: every sequence token by token.  chunk > 0: three passes over chunks of that many tokens; ws_state holds
 // max_chunks * N * channels floats and ws_steps max_chunks * channels, max_chunks >= sum over the sequences of
 // ceil(q_len / chunk).
-PLLM_API int pllm_selective_scan(int dtype, const void* x, long x_stride, const float* raw, float* dt, const float* dt_bias, const float* bc, long bc_stride,
+PLLM_API int pllm_selective_scan(int dtype, const void* x, long x_stride, const float* raw, float* dt, const float* dt_bias, const void* bc, long bc_stride,
                                  const float* a2, const float* skip, const void* z, long z_stride, float* state, long slot_stride,
                                  const int* state_slots, const int* seq_starts, const int* cu_seqlens, void* out, int num_seqs, int channels,
                                  int N, int chunk, int max_chunks, float* ws_state, float* ws_steps, hipStream_t stream) {
@@ -202,15 +210,15 @@ PLLM_API int pllm_selective_scan(int dtype, const void* x, long x_stride, const 
   ScanArgs a{x, x_stride, raw, dt, dt_bias, a2, skip, z, z_stride, state, slot_stride, state_slots, seq_starts, cu_seqlens, out,
              channels, N, num_seqs, chunk, ws_state, ws_steps};
   if (chunk == 0) {
-    if (dtype == PLLM_F32) launch_scan<float, kScanWhole>(a, bc, bc_stride, num_seqs, stream);
-    else launch_scan<bf16, kScanWhole>(a, bc, bc_stride, num_seqs, stream);
+    if (dtype == PLLM_F32) launch_scan<float, float, kScanWhole>(a, bc, bc_stride, num_seqs, stream);
+    else launch_scan<bf16, bf16, kScanWhole>(a, bc, bc_stride, num_seqs, stream);
     PLLM_RETURN_LAST_ERROR();
   }
   const size_t per_seq = (size_t)N * channels;
-  if (dtype == PLLM_F32) launch_scan<float, kScanState>(a, bc, bc_stride, max_chunks, stream);
-  else launch_scan<bf16, kScanState>(a, bc, bc_stride, max_chunks, stream);
+  if (dtype == PLLM_F32) launch_scan<float, float, kScanState>(a, bc, bc_stride, max_chunks, stream);
+  else launch_scan<bf16, float, kScanState>(a, bc, bc_stride, max_chunks, stream);
   hipLaunchKernelGGL(selective_scan_carry_kernel, dim3((unsigned)((per_seq + 255) / 256), num_seqs), dim3(256), 0, stream, a);
-  if (dtype == PLLM_F32) launch_scan<float, kScanOut>(a, bc, bc_stride, max_chunks, stream);
-  else launch_scan<bf16, kScanOut>(a, bc, bc_stride, max_chunks, stream);
+  if (dtype == PLLM_F32) launch_scan<float, float, kScanOut>(a, bc, bc_stride, max_chunks, stream);
+  else launch_scan<bf16, float, kScanOut>(a, bc, bc_stride, max_chunks, stream);
   PLLM_RETURN_LAST_ERROR();
 }

@@ -26,7 +26,7 @@
 //
 // One workgroup barrier per stage (an s_barrier alone: it does not wait for loads under way, so the weights keep
 // streaming across it).  At the end the eight wavefronts' sums are added through LDS in wavefront order and the epilogue
-// runs: bfloat16 or float out, act(gate) * up, the rotary encoding of q and k with the write of k and v into their cache
+// runs: bfloat16 or float out, act(row), act(gate) * up, the rotary encoding of q and k with the write of k and v into their cache
 // pages, or float partial sums of a range of K ([splits, M, N]: matrices with few rows are cut along K so that every
 // compute unit streams; whoever consumes them adds the ranges in order).
 // Every output element is summed in one fixed order that does not depend on the number of rows.
@@ -43,7 +43,7 @@ constexpr int kChunkK = 32;                          // columns of one matrix in
 constexpr int kStageK = kComputeWaves * kChunkK;     // 256
 constexpr int kTileElems = 16 * kChunkK;             // 512 elements, 1 KB
 
-enum { SL_BF16 = 0, SL_F32 = 1, SL_GATED = 2, SL_PARTIAL = 3, SL_ROPE_KV = 4 };
+enum { SL_BF16 = 0, SL_F32 = 1, SL_GATED = 2, SL_PARTIAL = 3, SL_ROPE_KV = 4, SL_ACT = 5 };
 
 struct StreamLinearParams {
   const bf16* x; int ldx;
@@ -58,6 +58,7 @@ struct StreamLinearParams {
   const int* positions; const float* cos_t; const float* sin_t; const int* slots;
   bf16* k_pages; bf16* v_pages;
   int num_heads, num_kv_heads, head_dim, block_size;
+  float act_p0, act_p1;       // SL_ACT: the activation's parameters (`activation` is one of PLLM_ROW_ACT_* then)
 };
 
 template <int N_>
@@ -252,10 +253,10 @@ __global__ __launch_bounds__(kStreamThreads) void stream_linear_kernel(const Str
       }
     } else {
       const int n = unit * 16 + g * 4;
-      if (EPI == SL_BF16) {
+      if (EPI == SL_BF16 || EPI == SL_ACT) {
         bf16 o[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = __float2bfloat16(a[i]);
+        for (int i = 0; i < 4; ++i) o[i] = __float2bfloat16(EPI == SL_ACT ? row_activation(a[i], p.activation, p.act_p0, p.act_p1) : a[i]);
         bf16* dst = (bf16*)p.out + (size_t)m * p.ldo + n;
         if (n + 3 < p.N && (p.ldo & 3) == 0) *reinterpret_cast<uint2*>(dst) = *reinterpret_cast<const uint2*>(o);
         else {
@@ -296,7 +297,7 @@ PLLM_API int pllm_stream_linear_row_blocks(int M) { return (M + 127) / 128; }
 PLLM_API int pllm_stream_linear(int epi, const void* x, int ldx, const void* wt, void* out, int ldo, int M, int N, int K,
                                 int weight_blocks, int nt, int splits, const int* positions, const float* cos_t, const float* sin_t,
                                 const int* slots, void* k_pages, void* v_pages, int num_heads, int num_kv_heads, int head_dim,
-                                int block_size, int activation, hipStream_t stream) {
+                                int block_size, int activation, float act_p0, float act_p1, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
   if (K <= 0 || (K % kChunkK) || (ldx & 7) || nt < 1 || nt > 4 || weight_blocks <= 0 || (weight_blocks % 24) || splits < 1) return -2;
   if (splits > 1 && epi != SL_PARTIAL) return -2;
@@ -308,8 +309,8 @@ PLLM_API int pllm_stream_linear(int epi, const void* x, int ldx, const void* wt,
   p.x = (const bf16*)x; p.ldx = ldx; p.wt = (const bf16*)wt; p.out = out; p.ldo = ldo; p.M = M; p.N = N; p.K = K;
   p.positions = positions; p.cos_t = cos_t; p.sin_t = sin_t; p.slots = slots; p.k_pages = (bf16*)k_pages; p.v_pages = (bf16*)v_pages;
   p.num_heads = num_heads; p.num_kv_heads = num_kv_heads; p.head_dim = head_dim; p.block_size = block_size;
-  if (activation < 0 || activation >= PLLM_ACT_COUNT) return -2;
-  p.activation = activation;
+  if (activation < 0 || activation >= (epi == SL_ACT ? PLLM_ROW_ACT_COUNT : PLLM_ACT_COUNT)) return -2;
+  p.activation = activation; p.act_p0 = act_p0; p.act_p1 = act_p1;
   p.ksteps = K / kChunkK;
   p.num_stages = (K + kStageK - 1) / kStageK;
   p.stages_per_split = (p.num_stages + splits - 1) / splits;
@@ -355,6 +356,7 @@ PLLM_API int pllm_stream_linear(int epi, const void* x, int ldx, const void* wt,
     case SL_GATED: PLLM_SL_SHAPES(SL_GATED); break;
     case SL_PARTIAL: PLLM_SL_SHAPES(SL_PARTIAL); break;
     case SL_ROPE_KV: PLLM_SL_SHAPES(SL_ROPE_KV); break;
+    case SL_ACT: PLLM_SL_SHAPES(SL_ACT); break;
   }
 #undef PLLM_SL_SHAPES
 #undef PLLM_SL

@@ -10,7 +10,7 @@ import torch
 
 from ..csrc import ops
 from .base import FeedForward
-from .linear import Weight, gated_linear, linear
+from .linear import Weight, activated_linear, gated_linear, linear
 from .registry import BuildEnv, register_feed_forward
 from .spec import WeightSpec
 
@@ -103,7 +103,7 @@ class PlainMLP(FeedForward):
         self._w.clear()
 
     def forward(self, h, ctx):
-        act = ops.activate_rows(linear(h, self.w_up), self.activation, self.act_params)
+        act = activated_linear(h, self.w_up, self.activation, self.act_params)
         if getattr(ctx, "float_branch", False):
             return linear(act, self.w_down, out_dtype=torch.float32)
         return linear(act, self.w_down, partial_ok=bool(getattr(ctx, "partial_sums_ok", False)))

@@ -114,7 +114,7 @@ def _streams(x, weight, epi: int, partial_ok: bool = False) -> bool:
     return _few_weight_rows(weight) and (k < STREAM_LONG_K or rows <= STREAM_LONG_K_MAX_ROWS or (partial_ok and epi == ops.SL_BF16))
 
 
-def _stream(x, weight: Weight, epi: int, rope: dict | None = None, partial_ok: bool = False, activation: str = "silu"):
+def _stream(x, weight: Weight, epi: int, rope: dict | None = None, partial_ok: bool = False, activation: str = "silu", act_params: tuple = (0.0, 0.0)):
     x = rows_of(x)
     if x.stride(1) != 1 or x.stride(0) % 8 or x.data_ptr() % 16:
         x = x.contiguous()
@@ -125,13 +125,13 @@ def _stream(x, weight: Weight, epi: int, rope: dict | None = None, partial_ok: b
         nt, splits = ops.stream_linear_plan(x.shape[0], n, k, ops._num_compute_units(x.device), partial=True)
         if splits > 1:
             return ops.stream_linear(x, weight.tiled, ops.SL_PARTIAL, nt=nt, splits=splits)
-    return ops.stream_linear(x, weight.tiled, epi, rope=rope)
+    return ops.stream_linear(x, weight.tiled, epi, rope=rope, activation=activation, act_params=act_params)
 
 
 _PAIRING_OF = {ops.EPI_GATED: "gated", ops.EPI_ROPE_KV: "rotary"}
 
 
-def _fused(x, weight, epi: int, rope: dict | None = None, activation: str = "silu"):
+def _fused(x, weight, epi: int, rope: dict | None = None, activation: str = "silu", act_params: tuple = (0.0, 0.0)):
     """The fused decode kernel if it takes the operands, else None.  With a ``Weight`` whose tiled copy has the pairing
     of the epilogue, products of at most 16 rows with the sum and norm in front stream the weights from that copy
     (11264 x 2048: 12.3 against 13.4 us; 2560 x 2048 with the rotary epilogue: 7.4 against 7.9; 32000 x 2048: 29.0 against 30.4)."""
@@ -143,7 +143,7 @@ def _fused(x, weight, epi: int, rope: dict | None = None, activation: str = "sil
     if isinstance(x, PendingNorm):
         if x.fusable() and ops.decode_linear_takes(x.num_rows, x.x.shape[1], x.x, weight):
             args = x.fused_arguments()
-            out = ops.decode_linear(x.x, weight, epi, rope=rope, tiled=tiled, activation=activation, **args)
+            out = ops.decode_linear(x.x, weight, epi, rope=rope, tiled=tiled, activation=activation, act_params=act_params, **args)
             x.fused_done(args)
             return out
         x = x.rows()
@@ -151,7 +151,7 @@ def _fused(x, weight, epi: int, rope: dict | None = None, activation: str = "sil
             and ops.decode_linear_pays(x.shape[0], weight.shape[0], x.shape[1], epi, staged=False)):
         # (plain rows keep the row-major matrix: from the tiled copy 4096 x 4096 and 4096 x 14336 took 10.7 and 32.9 us at 8
         #  rows against 9.3 and 27.7, and the smaller matrices the same time either way)
-        return ops.decode_linear(x, weight, epi, rope=rope, activation=activation)
+        return ops.decode_linear(x, weight, epi, rope=rope, activation=activation, act_params=act_params)
     return None
 
 
@@ -245,6 +245,19 @@ def gated_linear(x, w_gate_up, activation: str = "silu") -> torch.Tensor:
             return out
     w_gate_up = _plain(w_gate_up)
     return ops.gate_mul(linear(x, w_gate_up), activation)
+
+
+def activated_linear(x, weight, activation: str, act_params: tuple = (0.0, 0.0)) -> torch.Tensor:
+    """act(x W^T) [T, N] in the compute type (a feed-forward without a gate): in the product's own kernel where the fused kernels for
+    few rows take it, else by a kernel behind the product.  ``activation``: one of ``ops.ROW_ACTIVATIONS`` with ``act_params``."""
+    x = _operand(x)
+    if _streams(x, weight, ops.SL_BF16) and weight.pairing == "plain":
+        return _stream(x, weight, ops.SL_ACT, activation=activation, act_params=act_params)
+    if weight.dtype == torch.bfloat16:
+        out = _fused(x, weight, ops.EPI_ACT, activation=activation, act_params=act_params)
+        if out is not None:
+            return out
+    return ops.activate_rows(linear(x, weight), activation, act_params)
 
 
 def qkv_rotary_cache(x, w_qkv, positions: torch.Tensor, position_encoding, num_heads: int, num_kv_heads: int,

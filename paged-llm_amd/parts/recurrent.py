@@ -319,9 +319,9 @@ class Hgrn2Mixer(_StatefulMixer):
 class Mamba1Mixer(_StatefulMixer):
     """A selective scan:  [x | z] = W_in h; x passes a causal convolution per channel (with bias) and SiLU;  [low | B | C] = W_x x,
     dt = softplus(W_dt low + b);  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n with A = -exp(A_log),
-    y_c = sum_n S[c, n] C_n + D_c x_c;  then y silu(z), the output product.  Step sizes, decays, B, C and the state are float
-    whatever the compute type.  The state slot holds S [N, inner] (N padded to a size the kernel takes, the padding zero) and
-    behind it the convolution's last inputs.
+    y_c = sum_n S[c, n] C_n + D_c x_c;  then y silu(z), the output product.  Step sizes, decays, the state and its sums are float
+    whatever the compute type (the products that make them leave rows in it).  The state slot holds S [N, inner] (N padded to a
+    size the kernel takes, the padding zero) and behind it the convolution's last inputs.
 
     params: ``inner`` (channels), ``state`` (N), ``dt_rank``, ``conv`` (taps).  Tensors: ``in`` [2 inner, width], ``conv`` [inner,
     taps] with ``conv.b``, ``x`` [dt_rank + 2 N, inner], ``dt`` [inner, dt_rank] with ``dt.b``, ``A_log`` [inner, N], ``D`` [inner], ``o``."""
@@ -336,6 +336,7 @@ class Mamba1Mixer(_StatefulMixer):
             raise ValueError(f"a selective scan takes 1 to {ops.SCAN_STATE_MAX} state elements per channel; got {self.N}, {self.inner} channels, rank {self.rank}")
         self.dtype, self.device = env.dtype, env.device
         self.held = ops.scan_state_size(self.N)
+        self.low = -(-self.rank // 8) * 8                        # rows of the low-rank product, padded so that all three parts start on 16 bytes
         self.conv_at = self.held * self.inner
         self._w: dict = {}
         self.w_in = self.w_x = self.w_dt = self.w_o = self.a2 = None
@@ -348,10 +349,12 @@ class Mamba1Mixer(_StatefulMixer):
 
     def finalize(self):
         w, pad = self._w, self.held - self.N
-        self.w_in, self.w_dt, self.w_o = Weight(w.pop("in")), Weight(w.pop("dt")), Weight(w.pop("o"))
+        self.w_in, self.w_o = Weight(w.pop("in")), Weight(w.pop("o"))
         low, b, c = w.pop("x").split([self.rank, self.N, self.N], dim=0)
         zeros = b.new_zeros((pad, self.inner))
-        self.w_x = Weight(torch.cat([low, b, zeros, c, zeros], dim=0).contiguous())
+        self.w_x = Weight(torch.cat([low, b.new_zeros((self.low - self.rank, self.inner)), b, zeros, c, zeros], dim=0).contiguous())
+        dt = w.pop("dt")
+        self.w_dt = Weight(torch.cat([dt, dt.new_zeros((self.inner, self.low - self.rank))], dim=1).contiguous())
         a2 = torch.zeros((self.held, self.inner), dtype=torch.float32)
         a2[:self.N] = (-torch.exp(w.pop("A_log").double().cpu()) * math.log2(math.e)).T.float()      # A log2(e), one row per state element
         self.a2 = a2.to(self.device).contiguous()
@@ -364,12 +367,9 @@ class Mamba1Mixer(_StatefulMixer):
         proj = linear(h, self.w_in)
         seqs = (ctx.state_slots, ctx.seq_starts, ctx.cu_seqlens_q, ctx.num_seqs)
         x = ops.causal_conv(proj[:, :C], w["conv"], w["conv.b"], state, self.conv_at, *seqs, ctx.max_q_len)
-        low = linear(x, self.w_x, out_dtype=torch.float32)
-        step = low[:, :self.rank]
-        if self.dtype != torch.float32:
-            step = ops.activate_rows(step, None, out_dtype=self.dtype)
-        raw = linear(step, self.w_dt, out_dtype=torch.float32)
-        y = ops.selective_scan(x, raw, w["dt.b"], low[:, self.rank:], self.a2, w["D"], proj[:, C:], state, *seqs, max_q_len=ctx.max_q_len)
+        low = linear(x, self.w_x)
+        raw = linear(low[:, :self.low], self.w_dt, out_dtype=torch.float32)
+        y = ops.selective_scan(x, raw, w["dt.b"], low[:, self.low:], self.a2, w["D"], proj[:, C:], state, *seqs, max_q_len=ctx.max_q_len)
         return linear(y, self.w_o, out_dtype=_out_dtype(ctx))
 
 

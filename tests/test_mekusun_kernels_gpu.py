@@ -41,7 +41,7 @@ def test_selective_scan(channels, N, lengths, max_q, dtype):
     T, S, held = sum(lengths), len(lengths), ops.scan_state_size(N)
     x, z = rnd(T, channels).to(dtype), rnd(T, channels).to(dtype)
     raw, bias = rnd(T, channels), rnd(channels) - 2.0
-    B, C, D = rnd(T, N), rnd(T, N), rnd(channels)
+    B, C, D = rnd(T, N).to(dtype), rnd(T, N).to(dtype), rnd(channels)
     A = -torch.exp(rnd(channels, N) * 0.7)
     pad = lambda t: torch.cat([t, t.new_zeros(t.shape[0], held - N)], dim=1)
     a2 = torch.zeros(held, channels)
@@ -278,6 +278,21 @@ def test_activations_of_single_elements(name, cols, stride):
             # (a GELU far below zero is the difference of nearly equal numbers: absolute errors of z's own rounding there)
             err = ((got.double().cpu() - want).abs() / (want.abs() + 0.01 * x.to(src)[:, :cols].double().abs() + 1e-6)).max()
             assert float(err) < (2e-5 if out == torch.float32 else 5e-3), (name, src, out, float(err))
+
+
+@pytest.mark.parametrize("rows", [1, 5, 8, 16, 24, 40, 64, 128, 200])
+@pytest.mark.parametrize("name", ["xielu", "gelu"])
+def test_activation_in_the_products_kernel(rows, name):
+    """The product's own kernels for few and some rows, and the kernel behind the product, against the product in float64."""
+    from paged_llm_amd.parts.linear import Weight, activated_linear
+    gen = torch.Generator().manual_seed(rows)
+    for N, K in ((512, 256), (200, 1024)):
+        x, w = torch.randn(rows, K, generator=gen).bfloat16(), (torch.randn(N, K, generator=gen) * K ** -0.5).bfloat16()
+        got = activated_linear(dev(x), Weight(dev(w)), name, (0.8, 0.9))
+        z = x.double() @ w.double().T
+        want = plain.gelu_erf(z) if name == "gelu" else torch.where(z > 0, 0.8 * z * z, 0.9 * (torch.expm1(z.clamp(max=0)) - z.clamp(max=0))) + 0.5 * z
+        assert got.dtype == torch.bfloat16
+        close(got, want, 1e-2)
 
 
 def test_capped_logits():
