@@ -1,7 +1,7 @@
 // A matrix memory per head whose rows decay one by one and from which, token by token, a part of what the unit key reads is
 // removed along another direction:
 //   u = k / sqrt(sum(k^2) + 1e-6),   w = exp(-exp(-1/2) sigmoid(raw_w + w0)),   a = sigmoid(raw_a + bias_a)     per head and row
-//   S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T   (both terms read the old state),   o_t = S_t^T r,
+//   z = S^T u  (S as the token finds it),   S <- w . S - (a . u) z^T + k v^T  (w . S: row by row),   o = S^T r,
 // and behind it, per head, o / sqrt(mean(o^2) + eps) * weight * sigmoid(gate).
 //
 // A batch is token-major without padding: sequence s owns rows cu_seqlens[s] .. cu_seqlens[s + 1] - 1, its state sits in

@@ -1473,7 +1473,7 @@ SCAN_CHUNKS_FROM = 128            # tokens of the longest sequence of a step fro
 def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, bc: torch.Tensor, a2: torch.Tensor, skip: torch.Tensor,
                    z: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, seq_starts: torch.Tensor, cu_seqlens: torch.Tensor,
                    num_seqs: int, max_q_len: int = 0) -> torch.Tensor:
-    """S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,  y_c = sum_n S[c, n] C_n + skip_c x_c,  out = y silu(z), with
+    """s_c <- e^(dt_c A_c) * s_c + (dt_c x_c) B for the N states of channel c,  y_c = <s_c, C> + skip_c x_c,  out = y silu(z), with
     dt = softplus(raw_dt + dt_bias).  x, z [T, channels] (views of one type, unit inner stride), raw_dt contiguous float32
     [T, channels], bc [T, 2 N] of x's type (a view: B, then C; rows on 4-byte boundaries), a2 float32 [N, channels] = A log2(e) transposed, N as
     ``scan_state_size`` gives it; S float32 [N, channels] in front of ``state[slot]``; a sequence with seq_starts == 0 starts
@@ -1519,7 +1519,7 @@ def delta_rule(rows: torch.Tensor, columns: dict, raw_w: torch.Tensor, w0: torch
                heads: int, dim: int, state: torch.Tensor, state_slots: torch.Tensor, seq_starts: torch.Tensor, cu_seqlens: torch.Tensor,
                num_seqs: int, max_q_len: int = 0) -> torch.Tensor:
     """A matrix memory per head: u = k / sqrt(sum(k^2) + 1e-6), w = exp(-exp(-1/2) sigmoid(raw_w + w0)), a = sigmoid(raw_a +
-    bias_a), S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T, o_t = S_t^T r; then per head o / sqrt(mean(o^2) + eps) *
+    bias_a), z = S^T u, S <- w . S - (a . u) z^T + k v^T (w . S: row by row), o = S^T r; then per head o / sqrt(mean(o^2) + eps) *
     weight * sigmoid(gate).  ``rows`` [T, ...] holds r, k, v, raw_a and the gate, heads * dim columns each, from the columns
     ``columns`` = {"r", "k", "v", "a", "g"} on (unit inner stride); raw_w float32 [T, heads * dim]; w0, bias_a, weight float32
     [heads * dim].  S float32 [heads, dim, dim] in front of ``state[slot]``; a sequence with seq_starts == 0 starts from

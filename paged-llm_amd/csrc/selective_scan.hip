@@ -1,6 +1,6 @@
 // Selective scan: a recurrence with a state of N floats per channel whose decays depend on the token and the channel,
-//   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,   y_c = sum_n S[c, n] C_n + D_c x_c,
-// and the gate behind it, out = y silu(z).  The step sizes arrive raw: dt = softplus(raw + bias).
+//   s_c <- e^(step_c A_c) * s_c + (step_c x_c) B  for the N states s_c of channel c,   y_c = <s_c, C> + D_c x_c,
+// and the gate behind it, out = y silu(z).  The step sizes arrive raw: step = softplus(raw + bias).
 //
 // A batch is token-major without padding: sequence s owns rows cu_seqlens[s] .. cu_seqlens[s + 1] - 1, its state sits in
 // slot state_slots[s] as [N][channels] floats, and seq_starts[s] == 0 says that it starts now, from a zero state, whatever

@@ -26,7 +26,7 @@ Most are the same recurrence per head, S_t = a_t S_(t-1) + k_t (g_t v_t)^T, y_t 
 
 Two recurrences have kernels of their own:
 
-* ``mamba1`` (a selective scan, ``ops.selective_scan``): a state of N floats per channel whose decays exp(dt_c A[c, n]) differ
+* ``mamba1`` (a selective scan, ``ops.selective_scan``): a state of N floats per channel whose decays e^(step_c A_cn) differ
   from element to element, behind a short convolution; step sizes through a low-rank product, times silu(z), the output product.
 * ``general_delta`` (``ops.delta_rule``): a matrix memory whose rows decay one by one and from which, in front of every write, a
   part of what the unit key reads is removed along another direction; norm per head, weight, sigmoid gate, output product.
@@ -318,8 +318,8 @@ class Hgrn2Mixer(_StatefulMixer):
 
 class Mamba1Mixer(_StatefulMixer):
     """A selective scan:  [x | z] = W_in h; x passes a causal convolution per channel (with bias) and SiLU;  [low | B | C] = W_x x,
-    dt = softplus(W_dt low + b);  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n with A = -exp(A_log),
-    y_c = sum_n S[c, n] C_n + D_c x_c;  then y silu(z), the output product.  Step sizes, decays, the state and its sums are float
+    step = softplus(W_dt low + b);  s_c <- e^(step_c A_c) * s_c + (step_c x_c) B for channel c's vector of N states, with A = -e^(A_log);
+    y_c = <s_c, C> + D_c x_c;  then y silu(z), the output product.  Step sizes, decays, the state and its sums are float
     whatever the compute type (the products that make them leave rows in it).  The state slot holds S [N, inner] (N padded to a
     size the kernel takes, the padding zero) and behind it the convolution's last inputs.
 
@@ -376,7 +376,8 @@ class Mamba1Mixer(_StatefulMixer):
 class GeneralDeltaMixer(_StatefulMixer):
     """A generalized delta rule:  r = W_r h, k = W_k h, v = W_v h; a decay w = exp(-exp(-1/2) sigmoid(W_w2 tanh(W_w1 h) + w0)) and a
     removal rate a = sigmoid(W_a h + b_a) per head and key channel; with the unit key u = k / sqrt(sum(k^2) + 1e-6)
-    S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T  and  o_t = S_t^T r;  then each head's o divided by its root mean
+    the memory M [key, value] is read along u as it stands, z = M^T u, and becomes w . M - (a . u) z^T + k v^T (w . M: row by row);
+    o = M^T r;  then each head's o divided by its root mean
     square, times ``norm`` (over all heads' channels), times sigmoid(W_g h), the output product.  Decays, rates, unit keys, the
     state and the norm are float whatever the compute type.
 

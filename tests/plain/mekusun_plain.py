@@ -5,10 +5,10 @@ x <- x + s1 * N1b(mixer(N1(x))), x <- x + s2 * N2b(ff(N2(x))), with RMS norms wh
 scale s on what a sublayer adds.  Behind every layer the stream becomes a weighted sum over the embedding's output and
 the results of all layers up to this one, each result taken before that sum.  A layer holds one of three mixers:
 
-* ``mamba1``: a state per channel, S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n, behind a short convolution.
+* ``mamba1``: a vector of states per channel, s_c <- e^(dt_c A_c) * s_c + (dt_c x_c) B, behind a short convolution.
 * ``latent_attention``: keys and values from one normed latent per token, one rotated key part for all heads.
 * ``general_delta``: per head a matrix memory whose rows decay one by one and from which a part of what the unit key
-  reads is removed along another direction, S <- diag(w) S - (a u) (u^T S) + k v^T.
+  reads (z = S^T u) is removed along another direction, S <- w . S - (a . u) z^T + k v^T, row by row.
 
 and a dense feed-forward with a learned activation, or routed ungated experts.  The logits are capped by a tanh.
 Everything is computed in one floating type chosen by the caller.  It shares no code with the engine under
@@ -167,7 +167,7 @@ def latent_attention(h, w: dict, m: dict, eps: float, positions):
 
 
 def delta_memory(r, k, v, w, a):
-    """r, k, v, w, a [T, heads, d]: S <- diag(w) S - (a u) (u^T S) + k v^T with u the unit key, both terms from the old S;
+    """r, k, v, w, a [T, heads, d]: z = S^T u with u the unit key, S <- w . S - (a . u) z^T + k v^T (w . S row by row);
     o = S^T r."""
     u = k / torch.sqrt((k * k).sum(-1, keepdim=True) + 1e-6)
     T, H, d = k.shape

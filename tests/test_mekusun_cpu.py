@@ -201,7 +201,7 @@ def test_mamba1_reads_its_parts_in_order():
 
 
 def test_delta_memory_as_products_of_transitions():
-    """S_t = (diag(w_t) - (a_t u_t) u_t^T) S_(t-1) + k_t v_t^T: the output as a sum over tokens of products of those matrices."""
+    """A token moves the memory by one matrix, diag(w) - (a . u) u^T, and adds k v^T: the output as a sum over tokens of products of those matrices."""
     torch.manual_seed(2)
     T, H, n = 8, 2, 4
     d = lambda *s: torch.randn(*s, dtype=torch.float64)
