@@ -4,7 +4,9 @@
 //   attn_prepare      per token and head, from the float sums of the q/k/v product: + bias, a short causal convolution
 //                     over time on every channel (inputs of earlier steps from the request's state slot), rotary
 //                     encoding of the first rot elements of q and k heads (pairs (i, i + rot/2) or (2i, 2i + 1)),
-//                     q and k divided by their root mean square over the head (unless qk_norm is 0), q written as rows of padded heads,
+//                     q and k divided by their root mean square over the head (unless qk_norm is 0), behind the rotation or
+//                     (norm_first) in front of it, and times a weight per element that all heads share (when given),
+//                     q written as rows of padded heads,
 //                     k and v written into their cache pages; the values as projected (v_mode 0), divided by their root
 //                     mean square over the head (1), or the keys as they were before their rotation, the product
 //                     holding no value columns at all (2);
@@ -31,7 +33,8 @@ __global__ __launch_bounds__(64) void attn_prepare_kernel(
     const float* __restrict__ proj, int ld, const float* __restrict__ bias, const float* __restrict__ conv_w, int taps,
     const float* __restrict__ state, size_t slot_stride, const int* __restrict__ state_slots, const int* __restrict__ seq_starts,
     const int* __restrict__ cu_seqlens, int num_seqs, const int* __restrict__ positions, const float* __restrict__ cos_table,
-    const float* __restrict__ sin_table, int rot, int interleaved, float eps, int qk_norm, int v_mode, int heads, int kv_heads, int d, int dv, int D,
+    const float* __restrict__ sin_table, int rot, int interleaved, float eps, int qk_norm, int norm_first,
+    const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, int v_mode, int heads, int kv_heads, int d, int dv, int D,
     T* __restrict__ q_out, const int* __restrict__ slot_mapping, T* __restrict__ k_pages, T* __restrict__ v_pages, int block_size) {
   __shared__ float vals[kPrepMaxHead];
   const int lane = threadIdx.x;
@@ -80,13 +83,28 @@ __global__ __launch_bounds__(64) void attn_prepare_kernel(
       }
     }
     x[r] = v;
-    if (e < kPrepMaxHead) vals[e] = v;
   }
+  // x <- x / sqrt(mean(x^2) + eps) (* w): over the head's `width` elements
+  auto unit_rms = [&](const float* w) {
+    float sq = 0.f;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (lane + 64 * r < width) sq = fmaf(x[r], x[r], sq);
+    const float inv = 1.f / sqrtf(wave_sum(sq) / (float)width + eps);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int e = lane + 64 * r;
+      x[r] *= w ? inv * (e < width ? w[e] : 0.f) : inv;
+    }
+  };
+  const float* norm_w = kind == 0 ? q_norm_w : k_norm_w;
+  if (kind < 2 && qk_norm && norm_first) unit_rms(norm_w);
+#pragma unroll
+  for (int r = 0; r < 4; ++r) vals[lane + 64 * r] = x[r];
   __syncthreads();
   if (kind < 2) {
     const int pos = positions[tok];
     const int half = rot >> 1;
-    float sq = 0.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int e = lane + 64 * r;
@@ -101,23 +119,10 @@ __global__ __launch_bounds__(64) void attn_prepare_kernel(
         if (low) rotate_pair(x[r], other, c, s, out_lo, out_hi); else rotate_pair(other, x[r], c, s, out_lo, out_hi);
         x[r] = low ? out_lo : out_hi;
       }
-      if (e < width) sq = fmaf(x[r], x[r], sq);
     }
-    if (qk_norm) {
-      const float inv = 1.f / sqrtf(wave_sum(sq) / (float)width + eps);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) x[r] *= inv;
-    }
+    if (qk_norm && !norm_first) unit_rms(norm_w);
   }
-  if (kind == 2 && v_mode == 1) {
-    float sq = 0.f;
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      if (lane + 64 * r < width) sq = fmaf(x[r], x[r], sq);
-    const float inv = 1.f / sqrtf(wave_sum(sq) / (float)width + eps);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) x[r] *= inv;
-  }
+  if (kind == 2 && v_mode == 1) unit_rms(nullptr);
   if (kind == 0) {
     T* out = q_out + ((size_t)tok * heads + head) * D;
 #pragma unroll
@@ -177,7 +182,8 @@ __global__ __launch_bounds__(256) void conv_inputs_keep_kernel(
 PLLM_API int pllm_attn_prepare(int dtype, const float* proj, int ld, const float* bias, const float* conv_w, int taps, float* state,
                                long slot_stride, const int* state_slots, const int* seq_starts, const int* cu_seqlens, int num_seqs,
                                const int* positions, const float* cos_table, const float* sin_table, int rot, int interleaved,
-                               float eps, int qk_norm, int v_mode, int heads, int kv_heads, int d, int dv, int D, void* q_out, const int* slot_mapping,
+                               float eps, int qk_norm, int norm_first, const float* q_norm_w, const float* k_norm_w, int v_mode, int heads, int kv_heads,
+                               int d, int dv, int D, void* q_out, const int* slot_mapping,
                                void* k_pages, void* v_pages, int block_size, int num_tokens, hipStream_t stream) {
   if (num_tokens <= 0) return 0;
   if (d <= 0 || dv <= 0 || d > D || dv > D || D > kPrepMaxHead || rot < 0 || rot > d || (rot & 1) || taps > kPrepMaxTaps) return -2;
@@ -188,8 +194,8 @@ PLLM_API int pllm_attn_prepare(int dtype, const float* proj, int ld, const float
   dim3 grid(num_tokens, heads + (write ? 2 * kv_heads : 0)), block(64);
 #define PLLM_PREP(T)                                                                                                              \
   hipLaunchKernelGGL(attn_prepare_kernel<T>, grid, block, 0, stream, proj, ld, bias, conv_w, taps, state, (size_t)slot_stride,   \
-                     state_slots, seq_starts, cu_seqlens, num_seqs, positions, cos_table, sin_table, rot, interleaved, eps, qk_norm, v_mode, heads, \
-                     kv_heads, d, dv, D, (T*)q_out, slot_mapping, (T*)k_pages, (T*)v_pages, block_size)
+                     state_slots, seq_starts, cu_seqlens, num_seqs, positions, cos_table, sin_table, rot, interleaved, eps, qk_norm, norm_first, \
+                     q_norm_w, k_norm_w, v_mode, heads, kv_heads, d, dv, D, (T*)q_out, slot_mapping, (T*)k_pages, (T*)v_pages, block_size)
   if (dtype == PLLM_F32) PLLM_PREP(float); else PLLM_PREP(bf16);
 #undef PLLM_PREP
   if (taps > 1) {

@@ -34,11 +34,12 @@ __device__ __forceinline__ float gate_activation(float z, int act) {
 
 // An activation of single elements: of a feed-forward without a gate, or of a low-rank product's inner rows.  The first two
 // are the gate activations above; then GELU itself, 0.5 z (1 + erf(z / sqrt(2))); xIELU, p0 z^2 + z / 2 above zero and
-// p1 (exp(z) - 1 - z) + z / 2 below; tanh; and none.
-enum { PLLM_ROW_ACT_GELU = 2, PLLM_ROW_ACT_XIELU = 3, PLLM_ROW_ACT_TANH = 4, PLLM_ROW_ACT_NONE = 5, PLLM_ROW_ACT_COUNT = 6 };
+// p1 (exp(z) - 1 - z) + z / 2 below; tanh; none; and the square of relu, max(z, 0)^2.
+enum { PLLM_ROW_ACT_GELU = 2, PLLM_ROW_ACT_XIELU = 3, PLLM_ROW_ACT_TANH = 4, PLLM_ROW_ACT_NONE = 5, PLLM_ROW_ACT_RELU2 = 6, PLLM_ROW_ACT_COUNT = 7 };
 
 __device__ __forceinline__ float row_activation(float z, int act, float p0 = 0.f, float p1 = 0.f) {
   if (act < PLLM_ACT_COUNT) return gate_activation(z, act);
+  if (act == PLLM_ROW_ACT_RELU2) { const float u = fmaxf(z, 0.f); return u * u; }
   if (act == PLLM_ROW_ACT_GELU) return 0.5f * z * (1.f + erff(z * 0.7071067811865476f));
   if (act == PLLM_ROW_ACT_XIELU) return fmaf(z > 0.f ? p0 * z : p1, z > 0.f ? z : expm1f(z) - z, 0.5f * z);
   return act == PLLM_ROW_ACT_TANH ? tanhf(z) : z;

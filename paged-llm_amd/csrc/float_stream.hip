@@ -134,10 +134,63 @@ __global__ void layernorm_kernel(const TI* __restrict__ in, const int* __restric
 }
 
 // The same with the row in registers, four elements per thread and load (hidden a multiple of 4 up to kRowRegs * 1024,
-// rows on 16-byte boundaries in float and 8-byte ones in bfloat16): every value is read once.
+// rows on 16-byte boundaries in float and 8-byte ones in bfloat16): every value is read once, and the stream's row, the
+// weight and the bias are asked for before the first sum.
 constexpr int kRowRegs = 4;
 
 template <typename T> struct alignas(4 * sizeof(T)) Quad { T v[4]; };
+
+struct HeldRow { float x[kRowRegs][4]; };
+
+__device__ __forceinline__ void load_held(HeldRow& d, const float* p, int hidden) {
+#pragma unroll
+  for (int j = 0; j < kRowRegs; ++j) {
+    const int at = (j * 256 + threadIdx.x) * 4;
+    if (at < hidden) {
+      const float4 v = *reinterpret_cast<const float4*>(p + at);
+      d.x[j][0] = v.x; d.x[j][1] = v.y; d.x[j][2] = v.z; d.x[j][3] = v.w;
+    }
+  }
+}
+
+// v: the row that is normed.  stream_row / out_row: the row's places in the stream (its values in `add`) and in the output, or null.
+template <typename TO>
+__device__ __forceinline__ void layernorm_held(const HeldRow& v, const HeldRow& add, const HeldRow& w, const HeldRow& b, float eps,
+                                               float* stream_row, TO* out_row, int hidden, float* scratch) {
+  float acc = 0.f;
+#pragma unroll
+  for (int j = 0; j < kRowRegs; ++j)
+    if ((j * 256 + (int)threadIdx.x) * 4 < hidden) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc += v.x[j][e];
+    }
+  const float mean = block_sum(acc, scratch) / (float)hidden;
+  float sq = 0.f;
+#pragma unroll
+  for (int j = 0; j < kRowRegs; ++j)
+    if ((j * 256 + (int)threadIdx.x) * 4 < hidden) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) { const float d = v.x[j][e] - mean; sq = fmaf(d, d, sq); }
+    }
+  const float var = block_sum(sq, scratch) / (float)hidden;
+  const float inv = 1.f / sqrtf(var + eps);
+#pragma unroll
+  for (int j = 0; j < kRowRegs; ++j) {
+    const int at = (j * 256 + threadIdx.x) * 4;
+    if (at < hidden) {
+      float y[4];
+      Quad<TO> o;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        y[e] = (v.x[j][e] - mean) * inv * w.x[j][e] + b.x[j][e];
+        if (stream_row) y[e] += add.x[j][e];
+        o.v[e] = from_f32<TO>(y[e]);
+      }
+      if (stream_row) *reinterpret_cast<float4*>(stream_row + at) = make_float4(y[0], y[1], y[2], y[3]);
+      if (out_row) *reinterpret_cast<Quad<TO>*>(out_row + at) = o;
+    }
+  }
+}
 
 template <typename TI, typename TO>
 __global__ __launch_bounds__(256) void layernorm_regs_kernel(const TI* __restrict__ in, const int* __restrict__ row_index,
@@ -147,51 +200,96 @@ __global__ __launch_bounds__(256) void layernorm_regs_kernel(const TI* __restric
   const int r = blockIdx.x;
   const size_t src = row_index ? (size_t)row_index[r] : (size_t)r;
   const TI* v = in + src * hidden;
-  float x[kRowRegs][4], add[kRowRegs][4];
-  float acc = 0.f;
+  float* stream_row = stream_rows ? stream_rows + (size_t)r * hidden : nullptr;
+  HeldRow x, add, ww, bb;
 #pragma unroll
   for (int j = 0; j < kRowRegs; ++j) {
     const int at = (j * 256 + threadIdx.x) * 4;
     if (at < hidden) {
       const Quad<TI> q = *reinterpret_cast<const Quad<TI>*>(v + at);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) { x[j][e] = to_f32(q.v[e]); acc += x[j][e]; }
-      if (stream_rows) {                                   // asked for early: it arrives while the sums are made
-        const float4 sv = *reinterpret_cast<const float4*>(stream_rows + (size_t)r * hidden + at);
-        add[j][0] = sv.x; add[j][1] = sv.y; add[j][2] = sv.z; add[j][3] = sv.w;
-      }
+      for (int e = 0; e < 4; ++e) x.x[j][e] = to_f32(q.v[e]);
     }
   }
-  const float mean = block_sum(acc, scratch) / (float)hidden;
-  float sq = 0.f;
+  if (stream_row) load_held(add, stream_row, hidden);
+  load_held(ww, w, hidden);
+  load_held(bb, b, hidden);
+  layernorm_held(x, add, ww, bb, eps, stream_row, rows ? rows + (size_t)r * hidden : nullptr, hidden, scratch);
+}
+
+// A branch that is a sum of experts' rows, formed by the kernel that would have read it: branch[r][i] = sum over k < top, in
+// order, of weights[r, k] * (row_of_pair[r, k] >= 0 ? expert_out[row_of_pair[r, k]][i] : h[r][i]).
+struct ChoiceSum {
+  const float* expert_out; const void* h; long ld_h; const int* row_of_pair; const float* weights; int top;
+};
+constexpr int kSumTop = 64, kSumAhead = 4;       // choices of a token at most; choices whose rows are asked for at once
+
+// The layer norm of such a sum, added to the stream: the kernel above with the choices' rows and weights read once per
+// workgroup into LDS and the rows of four choices asked for before the first of them is added.
+template <typename TO, typename TH>
+__global__ __launch_bounds__(256) void layernorm_sum_kernel(const ChoiceSum sum, const float* __restrict__ w, const float* __restrict__ b,
+                                                            float eps, float* stream_rows, TO* __restrict__ rows, int hidden) {
+  __shared__ float scratch[16];
+  __shared__ int row_s[kSumTop];
+  __shared__ float weight_s[kSumTop];
+  const int r = blockIdx.x;
+  float* stream_row = stream_rows + (size_t)r * hidden;
+  if ((int)threadIdx.x < sum.top) {
+    row_s[threadIdx.x] = sum.row_of_pair[(size_t)r * sum.top + threadIdx.x];
+    weight_s[threadIdx.x] = sum.weights[(size_t)r * sum.top + threadIdx.x];
+  }
+  HeldRow x, add, ww, bb;
+  load_held(add, stream_row, hidden);
+  load_held(ww, w, hidden);
+  load_held(bb, b, hidden);
+  __syncthreads();
+  const TH* own = reinterpret_cast<const TH*>(sum.h) + (size_t)r * sum.ld_h;
 #pragma unroll
   for (int j = 0; j < kRowRegs; ++j) {
     const int at = (j * 256 + threadIdx.x) * 4;
-    if (at < hidden) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) { const float d = x[j][e] - mean; sq = fmaf(d, d, sq); }
-    }
-  }
-  const float var = block_sum(sq, scratch) / (float)hidden;
-  const float inv = 1.f / sqrtf(var + eps);
+    for (int e = 0; e < 4; ++e) x.x[j][e] = 0.f;
+    if (at >= hidden) continue;
+    for (int k0 = 0; k0 < sum.top; k0 += kSumAhead) {
+      float4 v[kSumAhead];
 #pragma unroll
-  for (int j = 0; j < kRowRegs; ++j) {
-    const int at = (j * 256 + threadIdx.x) * 4;
-    if (at < hidden) {
-      const float4 wv = *reinterpret_cast<const float4*>(w + at), bv = *reinterpret_cast<const float4*>(b + at);
-      const float ww[4] = {wv.x, wv.y, wv.z, wv.w}, bb[4] = {bv.x, bv.y, bv.z, bv.w};
-      float y[4];
-      Quad<TO> o;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        y[e] = (x[j][e] - mean) * inv * ww[e] + bb[e];
-        if (stream_rows) y[e] += add[j][e];
-        o.v[e] = from_f32<TO>(y[e]);
+      for (int u = 0; u < kSumAhead; ++u) {
+        const int row = row_s[k0 + u < sum.top ? k0 + u : sum.top - 1];
+        if (row >= 0) v[u] = *reinterpret_cast<const float4*>(sum.expert_out + (size_t)row * hidden + at);
+        else v[u] = make_float4(to_f32(own[at]), to_f32(own[at + 1]), to_f32(own[at + 2]), to_f32(own[at + 3]));
       }
-      if (stream_rows) *reinterpret_cast<float4*>(stream_rows + (size_t)r * hidden + at) = make_float4(y[0], y[1], y[2], y[3]);
-      if (rows) *reinterpret_cast<Quad<TO>*>(rows + (size_t)r * hidden + at) = o;
+#pragma unroll
+      for (int u = 0; u < kSumAhead; ++u)
+        if (k0 + u < sum.top) {
+          const float wt = weight_s[k0 + u];
+          x.x[j][0] = fmaf(wt, v[u].x, x.x[j][0]);
+          x.x[j][1] = fmaf(wt, v[u].y, x.x[j][1]);
+          x.x[j][2] = fmaf(wt, v[u].z, x.x[j][2]);
+          x.x[j][3] = fmaf(wt, v[u].w, x.x[j][3]);
+        }
     }
   }
+  layernorm_held(x, add, ww, bb, eps, stream_row, rows ? rows + (size_t)r * hidden : nullptr, hidden, scratch);
+}
+
+// Whether that kernel takes rows of this size and sums of so many choices (the caller forms the sum apart where not).
+PLLM_API int pllm_layernorm_sum_takes(int hidden, int top) { return hidden > 0 && hidden % 4 == 0 && hidden <= kRowRegs * 1024 && top > 0 && top <= kSumTop; }
+
+// out_dtype / h_dtype: the types of `rows` and of the tokens' own rows; every pointer to floats on a 16-byte boundary.
+PLLM_API int pllm_layernorm_sum(int out_dtype, int h_dtype, const float* expert_out, const void* h, long ld_h, const int* row_of_pair,
+                                const float* weights, int top, const float* w, const float* b, float eps, float* stream_rows, void* rows,
+                                int num_rows, int hidden, hipStream_t stream) {
+  if (num_rows <= 0) return 0;
+  if (!pllm_layernorm_sum_takes(hidden, top) || !stream_rows) return -2;
+  if ((uintptr_t)expert_out % 16 || (uintptr_t)w % 16 || (uintptr_t)b % 16 || (uintptr_t)stream_rows % 16 || (uintptr_t)rows % 16) return -2;
+  const ChoiceSum sum{expert_out, h, ld_h, row_of_pair, weights, top};
+  dim3 grid(num_rows), block(256);
+#define PLLM_LNS(TO, TH) \
+  hipLaunchKernelGGL((layernorm_sum_kernel<TO, TH>), grid, block, 0, stream, sum, w, b, eps, stream_rows, (TO*)rows, hidden)
+  if (out_dtype == PLLM_F32) { if (h_dtype == PLLM_F32) PLLM_LNS(float, float); else PLLM_LNS(float, bf16); }
+  else { if (h_dtype == PLLM_F32) PLLM_LNS(bf16, float); else PLLM_LNS(bf16, bf16); }
+#undef PLLM_LNS
+  PLLM_RETURN_LAST_ERROR();
 }
 
 // in_dtype / out_dtype: PLLM_F32 or PLLM_BF16.
@@ -304,12 +402,8 @@ __global__ __launch_bounds__(256) void rms_sandwich_kernel(const float* __restri
 // The same with a branch, for rows of up to 4,096 elements that 256 threads hold in registers (16 each): everything a
 // row needs (branch and bias, the stream's row, both weights) is asked for before the first sum, so the kernel waits
 // for memory once where the one above waits three times (decode steps: the weights have left the caches since the last
-// layer).  Elements, partial sums and their order are the ones of the kernel above.  The branch may still be a sum of
-// experts' rows (`sum.expert_out` set): branch[r][i] = sum over k < top, in order, of weights[r, k] * (row_of_pair[r, k]
-// >= 0 ? expert_out[row_of_pair[r, k]][i] : h[r][i]), formed here instead of by a kernel of its own.
-struct ChoiceSum {
-  const float* expert_out; const void* h; long ld_h; const int* row_of_pair; const float* weights; int top;
-};
+// layer).  Elements, partial sums and their order are the ones of the kernel above.  The branch may be a sum of
+// experts' rows (`sum.expert_out` set), formed here instead of by a kernel of its own.
 constexpr int kHeldPerThread = 16, kHeldThreads = 256;
 
 template <typename TO, typename TH>
@@ -732,7 +826,6 @@ __global__ __launch_bounds__(256) void dyt_sum_kernel(const float* __restrict__ 
 // The same with four elements per thread and load, the choices' rows and weights read once per workgroup into LDS and
 // the rows of four choices asked for before the first of them is added (hidden a multiple of 4, at most kSumTop choices,
 // rows on 16-byte boundaries): the loads of a step no longer wait for one another.
-constexpr int kSumTop = 64, kSumAhead = 4;
 
 template <typename TO, typename TH>
 __global__ __launch_bounds__(256) void dyt_sum_vec_kernel(const float* __restrict__ expert_out, const TH* __restrict__ h, long ld_h,

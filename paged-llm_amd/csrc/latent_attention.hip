@@ -17,7 +17,8 @@
 //                     behind where their latent-space parts go in the query rows [T, heads, width];
 //   latent_attention  for latents wider than those kernels take: one wavefront per (token, head), softmax over the
 //                     visible keys (causal, inside the window when there is one), keys walked in tiles of 64 aligned
-//                     to absolute positions, so that the order of every sum is the same however the tokens were cut.
+//                     to absolute positions, so that the order of every sum is the same however the tokens were cut; a
+//                     logit per head may take part in the softmax's sum (a key without a value).
 // All arithmetic is float; T is the storage type.
 #include "common.h"
 
@@ -116,7 +117,7 @@ template <typename T>
 __global__ __launch_bounds__(64) void latent_attention_kernel(
     const T* __restrict__ q, const T* __restrict__ k_pages, T* __restrict__ out, const int* __restrict__ block_tables,
     int bt_stride, const int* __restrict__ cu_seqlens_q, const int* __restrict__ seq_lens_k, int num_seqs, int heads,
-    int rank, int rot, int width, int block_size, float scale, int window) {
+    int rank, int rot, int width, int block_size, float scale, int window, const float* __restrict__ sinks) {
   __shared__ float q_s[kMaxRank + kMaxRot];
   __shared__ float p_s[64];
   __shared__ int slot_s[64];
@@ -143,6 +144,7 @@ __global__ __launch_bounds__(64) void latent_attention_kernel(
 #pragma unroll
   for (int r = 0; r < kPerLane; ++r) acc[r] = 0.f;
   float m = -INFINITY, l = 0.f;
+  if (sinks) { m = sinks[head]; l = 1.f; }             // as if one key with this score and no value had been seen
 
   for (int n0 = (first_key / 64) * 64; n0 <= q_pos; n0 += 64) {
     const int n = n0 + lane;
@@ -157,7 +159,7 @@ __global__ __launch_bounds__(64) void latent_attention_kernel(
       s = dot * scale;
     }
     const float m_new = fmaxf(m, wave_max(s));   // finite: the tile holds at least one visible key
-    const float alpha = expf(m - m_new);          // 0 on the first tile
+    const float alpha = expf(m - m_new);          // 0 on the first tile (without a sink)
     const float p = visible ? expf(s - m_new) : 0.f;
     l = l * alpha + wave_sum(p);
     m = m_new;
@@ -189,15 +191,15 @@ __global__ __launch_bounds__(64) void latent_attention_kernel(
 PLLM_API int pllm_latent_attention(int dtype, const void* q, const void* k_pages, void* out, const int* block_tables,
                                    int bt_stride, const int* cu_seqlens_q, const int* seq_lens_k, int num_seqs, int total_q,
                                    int heads, int rank, int rot, int width, int block_size, float scale, int window,
-                                   hipStream_t stream) {
+                                   const float* sinks, hipStream_t stream) {
   if (total_q <= 0 || num_seqs <= 0) return 0;
   if (rank <= 0 || rank > kMaxRank || rot < 0 || rot > kMaxRot || heads <= 0 || block_size <= 0 || width < rank + rot) return -2;
   dim3 grid(total_q, heads), block(64);
   if (dtype == PLLM_F32)
     hipLaunchKernelGGL(latent_attention_kernel<float>, grid, block, 0, stream, (const float*)q, (const float*)k_pages, (float*)out,
-                       block_tables, bt_stride, cu_seqlens_q, seq_lens_k, num_seqs, heads, rank, rot, width, block_size, scale, window);
+                       block_tables, bt_stride, cu_seqlens_q, seq_lens_k, num_seqs, heads, rank, rot, width, block_size, scale, window, sinks);
   else
     hipLaunchKernelGGL(latent_attention_kernel<bf16>, grid, block, 0, stream, (const bf16*)q, (const bf16*)k_pages, (bf16*)out,
-                       block_tables, bt_stride, cu_seqlens_q, seq_lens_k, num_seqs, heads, rank, rot, width, block_size, scale, window);
+                       block_tables, bt_stride, cu_seqlens_q, seq_lens_k, num_seqs, heads, rank, rot, width, block_size, scale, window, sinks);
   PLLM_RETURN_LAST_ERROR();
 }

@@ -21,13 +21,13 @@ constexpr int kMoeMaxTileRows = 128;  // ... and of the largest (steps with many
 
 // ---------------------------------------------------------------------------------------------
 // n = experts + pass-through experts router outputs; groups of n / groups neighbours; a group's mark is its largest
-// corrected score; only experts of the `keep` best groups can be chosen (ties: the lower index wins).
+// corrected score (mark_top 1) or the sum of its two largest (mark_top 2; of its only one where a group has one); only experts of the `keep` best groups can be chosen (ties: the lower index wins).
 constexpr int kRouteThreads = 1024, kRoutePieces = 16;   // threads of a workgroup in steps of few tokens; pieces the products are cut into
 
 template <typename T, int TOK>
 __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ router_w,
                                                                   const float* __restrict__ correction, int num_tokens, int width, int n_all,
-                                                                  int extra, int scoring, int groups, int keep, int top, int segments,
+                                                                  int extra, int scoring, int groups, int keep, int mark_top, int top, int segments,
                                                                   int* __restrict__ ids, float* __restrict__ weights, float* __restrict__ extras) {
   extern __shared__ float lds[];
   // n_all rows of the router matrix: the first n = n_all - extra are the experts' (scores, the choice), the last `extra`
@@ -167,9 +167,13 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
   if (keep < groups) {
     if (chooser)
       for (int g = lane; g < groups; g += 64) {
-        float best = -INFINITY;
-        for (int e = g * per; e < (g + 1) * per; ++e) best = fmaxf(best, choice[e]);
-        mark[g] = best;
+        float best = -INFINITY, second = -INFINITY;
+        for (int e = g * per; e < (g + 1) * per; ++e) {
+          const float c = choice[e];
+          second = fmaxf(second, fminf(best, c));
+          best = fmaxf(best, c);
+        }
+        mark[g] = mark_top > 1 && per > 1 ? best + second : best;
       }
     __syncthreads();
     // the `keep` best groups are taken one by one (a taken group's mark becomes -inf); the others' experts are shut out
@@ -212,12 +216,12 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
 // n_all = n + extra rows of the router matrix; scoring 0: softmax over the n router outputs, 1: a sigmoid of each, 2: the
 // choice by the outputs + correction, weights = the softmax over the chosen ones' outputs + correction.
 PLLM_API int pllm_moe_route(int dtype, const void* h, int ld, const float* router_w, const float* correction, int num_tokens, int width,
-                            int n_all, int extra, int scoring, int groups, int keep, int top, int* ids, float* weights, float* extras,
+                            int n_all, int extra, int scoring, int groups, int keep, int mark_top, int top, int* ids, float* weights, float* extras,
                             hipStream_t stream) {
   if (num_tokens <= 0) return 0;
   const int n = n_all - extra;
   if (extra < 0 || (extra > 0 && !extras) || scoring < 0 || scoring > 2) return -2;
-  if (n <= 0 || groups <= 0 || n % groups || keep <= 0 || keep > groups || top <= 0 || top > (n / groups) * keep) return -2;
+  if (n <= 0 || groups <= 0 || n % groups || keep <= 0 || keep > groups || mark_top < 1 || mark_top > 2 || top <= 0 || top > (n / groups) * keep) return -2;
   // as many parts of the row as make 16 pieces (1, 2, 4, 8 or 16 parts), none shorter than 64 elements: by the router's
   // shape alone, so that a token's scores do not depend on the step it is in
   int segments = 1;
@@ -229,7 +233,7 @@ PLLM_API int pllm_moe_route(int dtype, const void* h, int ld, const float* route
   const size_t lds = lds_one * tok;
 #define PLLM_ROUTE(T, TOK, THREADS)                                                                                              \
   hipLaunchKernelGGL((moe_route_kernel<T, TOK>), dim3((num_tokens + TOK - 1) / TOK), dim3(THREADS), lds, stream, (const T*)h, ld, \
-                     router_w, correction, num_tokens, width, n_all, extra, scoring, groups, keep, top, segments, ids, weights, extras)
+                     router_w, correction, num_tokens, width, n_all, extra, scoring, groups, keep, mark_top, top, segments, ids, weights, extras)
   if (dtype == PLLM_F32) { if (tok == 8) PLLM_ROUTE(float, 8, 512); else if (tok == 4) PLLM_ROUTE(float, 4, 256); else PLLM_ROUTE(float, 1, kRouteThreads); }
   else { if (tok == 8) PLLM_ROUTE(bf16, 8, 512); else if (tok == 4) PLLM_ROUTE(bf16, 4, 256); else PLLM_ROUTE(bf16, 1, kRouteThreads); }
 #undef PLLM_ROUTE

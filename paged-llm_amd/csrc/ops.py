@@ -161,8 +161,8 @@ def activation_code(name: str) -> int:
     return ACTIVATIONS[name]
 
 
-# of single elements, without a gate (PLLM_ROW_ACT_* in common.h); "xielu" has two parameters
-ROW_ACTIVATIONS = {**ACTIVATIONS, "gelu": 2, "xielu": 3, "tanh": 4, None: 5}
+# of single elements, without a gate (PLLM_ROW_ACT_* in common.h); "xielu" has two parameters, "relu2" is max(z, 0)^2
+ROW_ACTIVATIONS = {**ACTIVATIONS, "gelu": 2, "xielu": 3, "tanh": 4, None: 5, "relu2": 6}
 
 
 def row_activation_code(name: str | None) -> int:
@@ -1224,13 +1224,39 @@ def embed_bigram(ids: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor, sc
     return x
 
 
+def layernorm_sum_takes(hidden: int, top: int) -> bool:
+    return bool(_fn("float_stream.hip", "pllm_layernorm_sum_takes", signature=[c_int, c_int])(hidden, top))
+
+
+def _layernorm_of_sum(branch: "ChoiceSum", weight, bias, eps, stream_rows, out_dtype) -> torch.Tensor | None:
+    """The layer norm of a sum of experts' rows that the norm's kernel forms itself, added to the stream."""
+    rows, H = stream_rows.shape
+    e, h, rp, wt = branch.checked(rows, H)
+    _on_gpu(weight, bias, stream_rows)
+    for t, what in ((weight, "weight"), (bias, "bias")):
+        _need(t.dtype == torch.float32 and t.shape == (H,) and t.is_contiguous(), f"layer norm {what} must be float32 [{H}]")
+    _need(stream_rows.dtype == torch.float32 and stream_rows.is_contiguous(), f"the stream must be contiguous float32 [{rows}, {H}]")
+    out = torch.empty((rows, H), dtype=out_dtype, device=stream_rows.device) if out_dtype is not None else None
+    sig = [c_int, c_int, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_int, c_void_p]
+    _check(_fn("float_stream.hip", "pllm_layernorm_sum", signature=sig)(
+        dtype_code(out_dtype or torch.float32), dtype_code(h.dtype), _ptr(e), _ptr(h), h.stride(0), _ptr(rp), _ptr(wt), wt.shape[1],
+        _ptr(weight), _ptr(bias), c_float(eps), _ptr(stream_rows), _ptr(out), rows, H, _stream()), "layernorm_sum")
+    return out
+
+
 def layernorm(v: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float, stream_rows: torch.Tensor | None = None,
               row_index: torch.Tensor | None = None, out_dtype: torch.dtype | None = None) -> torch.Tensor | None:
     """y = (v - mean) / sqrt(var + eps) * weight + bias over each row of ``v`` (float32 or bfloat16), in float.
 
     With ``stream_rows`` (float32, as many rows as are normed): stream_rows += y in place, and the return value is the
     new stream rounded to ``out_dtype`` (None when ``out_dtype`` is None).  Without it the return value is y in
-    ``out_dtype``.  ``row_index`` (int32) picks the rows of ``v`` that are normed."""
+    ``out_dtype``.  ``row_index`` (int32) picks the rows of ``v`` that are normed.  With a stream ``v`` may be a ``ChoiceSum``
+    (a weighted sum of experts' rows), which the kernel forms itself where it takes the sizes."""
+    if isinstance(v, ChoiceSum):
+        _need(stream_rows is not None and row_index is None, "a sum of experts' rows is a branch that enters the stream")
+        if v.plain and layernorm_sum_takes(stream_rows.shape[1], v.weights.shape[1]):
+            return _layernorm_of_sum(v, weight, bias, eps, stream_rows, out_dtype)
+        v = v.rows()
     _on_gpu(v, weight, bias, stream_rows, row_index)
     _need(v.dim() == 2 and v.is_contiguous(), "layernorm input must be contiguous [rows, hidden]")
     H = v.shape[1]
@@ -1265,27 +1291,40 @@ def round_rows(x: torch.Tensor) -> torch.Tensor:
 
 
 # ------------------------------------------------------------------------------------------- per-head products
-def gemm_heads(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
+class HeadMatrices:
+    """One matrix per head, [heads, N, K] as a checkpoint stores them, in the order ``gemm_heads`` reads: float32 as they are (the plain
+    kernel takes rows of K), bfloat16 with N innermost, [heads, K, N] contiguous.  (The vendor's batched bfloat16 product has
+    faulted on this hardware with a transposed view as its right operand: it is only ever given a contiguous one.)"""
+
+    __slots__ = ("data", "heads", "out_features", "in_features")
+
+    def __init__(self, w: torch.Tensor):
+        _need(w.dim() == 3 and w.dtype in _DTYPE_CODE, "head matrices: [heads, N, K], float32 or bfloat16")
+        self.heads, self.out_features, self.in_features = w.shape
+        self.data = (w.transpose(1, 2) if w.dtype == torch.bfloat16 else w).contiguous()
+
+
+def gemm_heads(a: torch.Tensor, w: HeadMatrices, out: torch.Tensor | None = None) -> torch.Tensor:
     """out[t, h, :] = w[h] a[t, h, :] for a [T, heads, K] (a view into wider rows is fine: unit inner stride, any row and
-    head strides) and w [heads, N, K] contiguous; float accumulation in ascending k.  Returns [T, heads, N], contiguous
+    head strides) and w one [N, K] matrix per head; float accumulation.  Returns [T, heads, N], contiguous
     unless ``out`` (a view of the same freedom) is given."""
-    _on_gpu(a, w, out)
-    _need(a.dim() == 3 and w.dim() == 3 and a.shape[1] == w.shape[0] and a.shape[2] == w.shape[2] and a.dtype == w.dtype,
-          f"gemm_heads shapes {tuple(a.shape)} {a.dtype} x {tuple(w.shape)} {w.dtype}")
-    _need(a.stride(2) == 1 and w.is_contiguous(), "gemm_heads: unit inner stride of the rows, contiguous matrices")
+    _on_gpu(a, w.data, out)
+    _need(a.dim() == 3 and a.shape[1] == w.heads and a.shape[2] == w.in_features and a.dtype == w.data.dtype,
+          f"gemm_heads shapes {tuple(a.shape)} {a.dtype} x {w.heads} of [{w.out_features}, {w.in_features}] {w.data.dtype}")
+    _need(a.stride(2) == 1, "gemm_heads: unit inner stride of the rows")
     T, heads, K = a.shape
-    N = w.shape[1]
+    N = w.out_features
     if out is None:
         out = torch.empty((T, heads, N), dtype=a.dtype, device=a.device)
     _need(out.shape == (T, heads, N) and out.stride(2) == 1 and out.dtype == a.dtype, "bad output for gemm_heads")
     if a.dtype == torch.bfloat16:
         # bfloat16: the vendor's batched product (as the other bfloat16 products of more than a few rows), straight into
         # the output's rows through views with the heads in front
-        torch.bmm(a.transpose(0, 1), w.transpose(1, 2), out=out.transpose(0, 1))
+        torch.bmm(a.transpose(0, 1), w.data, out=out.transpose(0, 1))
         return out
     sig = [c_int, c_int, c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_void_p, c_int, c_long, c_int, c_int, c_int, c_int, c_void_p]
     _check(_fn("gemm_generic.hip", "pllm_gemm_nt_batched", signature=sig)(
-        dtype_code(a.dtype), dtype_code(out.dtype), _ptr(a), a.stride(0), a.stride(1), _ptr(w), K, N * K, _ptr(out), out.stride(0), out.stride(1),
+        dtype_code(a.dtype), dtype_code(out.dtype), _ptr(a), a.stride(0), a.stride(1), _ptr(w.data), K, N * K, _ptr(out), out.stride(0), out.stride(1),
         T, N, K, heads, _stream()), "gemm_heads")
     return out
 
@@ -1714,10 +1753,12 @@ def latent_prepare(rows: torch.Tensor, down_at: int, positions: torch.Tensor, co
 
 
 def latent_attention(q: torch.Tensor, rank: int, rot: int, k_pages: torch.Tensor, block_tables: torch.Tensor, cu_seqlens_q: torch.Tensor,
-                     seq_lens_k: torch.Tensor, scale: float, window: int) -> torch.Tensor:
+                     seq_lens_k: torch.Tensor, scale: float, window: int, sinks: torch.Tensor | None = None) -> torch.Tensor:
     """softmax(q . key_n * scale) over the visible keys n (causal; the last ``window`` positions when window > 0), times
     c_n, the first ``rank`` elements of key row n: [T, heads, rank].  q [T, heads, width] contiguous rows [qa | q_rot | 0],
-    k_pages [pages, 1, block, width] rows [c | key part | 0].  For latents wider than the paged attention kernels take."""
+    k_pages [pages, 1, block, width] rows [c | key part | 0].  ``sinks`` (float32 [heads]): a logit per head that takes part in the
+    softmax's sum and in nothing else.  For latents wider than the paged attention kernels take."""
+    ScoreTerms(0.0, None, sinks).checked(q.shape[1], q.device)
     _on_gpu(q, k_pages, block_tables, cu_seqlens_q, seq_lens_k)
     _need(q.dim() == 3 and q.is_contiguous() and k_pages.dtype == q.dtype, "latent_attention: contiguous q [T, heads, width] of the pages' type")
     T, heads, width = q.shape
@@ -1729,10 +1770,10 @@ def latent_attention(q: torch.Tensor, rank: int, rot: int, k_pages: torch.Tensor
     _need(cu_seqlens_q.dtype == torch.int32 and cu_seqlens_q.numel() == S + 1 and seq_lens_k.dtype == torch.int32, "lengths: int32")
     out = torch.empty((T, heads, rank), dtype=q.dtype, device=q.device)
     sig = [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-           c_int, c_void_p]
+           c_int, c_void_p, c_void_p]
     _check(_fn("latent_attention.hip", "pllm_latent_attention", signature=sig)(
         dtype_code(q.dtype), _ptr(q), _ptr(k_pages), _ptr(out), _ptr(block_tables), block_tables.stride(0), _ptr(cu_seqlens_q),
-        _ptr(seq_lens_k), S, T, heads, rank, rot, width, k_pages.shape[2], c_float(scale), window, _stream()), "latent_attention")
+        _ptr(seq_lens_k), S, T, heads, rank, rot, width, k_pages.shape[2], c_float(scale), window, _ptr(sinks), _stream()), "latent_attention")
     return out
 
 
@@ -2002,7 +2043,7 @@ def attn_prepare(proj: torch.Tensor, bias: torch.Tensor | None, conv_w: torch.Te
                  state_slots, seq_starts, cu_seqlens, num_seqs: int, positions: torch.Tensor, cos: torch.Tensor | None,
                  sin: torch.Tensor | None, rot: int, interleaved: bool, eps: float, heads: int, kv_heads: int, d: int, dv: int, D: int,
                  dtype: torch.dtype, slot_mapping: torch.Tensor | None, k_pages: torch.Tensor | None, v_pages: torch.Tensor | None,
-                 qk_norm: bool = True, values: str = "projected") -> torch.Tensor:
+                 qk_norm: bool = True, values: str = "projected", norm_weights: tuple | None = None, norm_first: bool = False) -> torch.Tensor:
     """``values``: "projected" (the product's value columns as they are), "normed" (each value head divided by its root mean
     square, ``eps`` inside the root, no weight) or "keys" (the product has no value columns: a value head is its key head
     as projected, with the bias, before the rotation; dv == d).
@@ -2010,11 +2051,16 @@ def attn_prepare(proj: torch.Tensor, bias: torch.Tensor | None, conv_w: torch.Te
     + ``bias``; a causal convolution over time per channel with ``conv_w`` float32 [channels, taps], whose inputs of
     earlier steps lie in ``state[slot]`` as [taps - 1, channels] and are left there for the next step; rotary encoding
     of the first ``rot`` elements of every q and k head; q and k heads divided by their root mean square (``eps``
-    inside the root; not with ``qk_norm`` False); returns q as [T, heads * D] in ``dtype`` (heads padded with zeros to D) and writes k into
+    inside the root; not with ``qk_norm`` False), behind the rotation or, with ``norm_first``, in front of it, and times ``norm_weights``
+    = (of q, of k), float32 [d] each, shared by all heads, when given; returns q as [T, heads * D] in ``dtype`` (heads padded with zeros to D) and writes k into
     ``k_pages`` [pages, kv_heads, block, D] and v into ``v_pages`` [pages, kv_heads, D, block] at ``slot_mapping``."""
     _on_gpu(proj, bias, conv_w, state, positions, cos, sin, slot_mapping, k_pages, v_pages)
     _need(values in VALUE_MODES, f"values: one of {tuple(VALUE_MODES)}, got {values!r}")
     _need(values != "keys" or d == dv, "values that are the keys have the keys' size")
+    q_w, k_w = norm_weights if norm_weights is not None else (None, None)
+    _on_gpu(q_w, k_w)
+    for t in (q_w, k_w):
+        _need(t is None or (qk_norm and t.dtype == torch.float32 and t.shape == (d,) and t.is_contiguous()), f"weights of the q/k norm: float32 [{d}]")
     channels = (heads + kv_heads) * d + (0 if values == "keys" else kv_heads * dv)
     _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= channels, f"proj: float32 [T, >= {channels}]")
     T = proj.shape[0]
@@ -2045,12 +2091,13 @@ def attn_prepare(proj: torch.Tensor, bias: torch.Tensor | None, conv_w: torch.Te
         _need(slot_mapping.dtype == torch.int32 and slot_mapping.numel() == T and slot_mapping.is_contiguous(), "slot_mapping: int32 [T]")
     q = torch.empty((T, heads * D), dtype=dtype, device=proj.device)
     sig = [c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
-           c_int, c_int, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p]
+           c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+           c_int, c_int, c_void_p]
     _check(_fn("attention_prepare.hip", "pllm_attn_prepare", signature=sig)(
         dtype_code(dtype), _ptr(proj), proj.stride(0), _ptr(bias), _ptr(conv_w), taps, _ptr(state) if taps > 1 else None,
         state.stride(0) if taps > 1 else 0, _ptr(state_slots) if taps > 1 else None, _ptr(seq_starts) if taps > 1 else None,
         _ptr(cu_seqlens) if taps > 1 else None, num_seqs, _ptr(positions), _ptr(cos) if rot else None, _ptr(sin) if rot else None, rot,
-        int(bool(interleaved)), c_float(eps), int(bool(qk_norm)), VALUE_MODES[values], heads, kv_heads, d, dv, D, _ptr(q), _ptr(slot_mapping) if write else None,
+        int(bool(interleaved)), c_float(eps), int(bool(qk_norm)), int(bool(norm_first)), _ptr(q_w), _ptr(k_w), VALUE_MODES[values], heads, kv_heads, d, dv, D, _ptr(q), _ptr(slot_mapping) if write else None,
         _ptr(k_pages) if write else None, _ptr(v_pages) if write else None, bs, T, _stream()), "attn_prepare")
     return q
 
@@ -2077,14 +2124,15 @@ MOE_MAX_EXPERTS = 1024
 
 
 MOE_SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}
+MOE_GROUP_MARKS = {"largest": 1, "two_largest": 2}
 MOE_FORMS = {"down": 0, "gated": 1, "plain": 2}
 
 
 def moe_route(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor | None, groups: int, keep: int, top: int,
-              scoring: str = "softmax", extra: int = 0) -> tuple:
+              scoring: str = "softmax", extra: int = 0, group_mark: str = "largest") -> tuple:
     """(ids int32 [T, top], weights float32 [T, top]): router outputs h router_w^T in float, scores by a softmax over all of
     them or (``scoring`` "sigmoid") a sigmoid of each, the ``top`` largest of score + correction among the experts of the
-    ``keep`` best of ``groups`` groups of neighbours (a group's mark: its largest corrected score), weights = the chosen
+    ``keep`` best of ``groups`` groups of neighbours (a group's mark: its largest corrected score, or with ``group_mark`` "two_largest" the sum of its two largest), weights = the chosen
     experts' scores.  ``scoring`` "softmax_chosen": output + correction is what the choice looks at, and the weights are the softmax
     over the chosen experts' output + correction alone.  The last ``extra`` rows of ``router_w`` are no experts: their outputs come back as they are, as a
     third result float32 [T, extra] (further products of the same rows that ride along)."""
@@ -2093,6 +2141,7 @@ def moe_route(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor 
     T, W = h.shape
     n_all = router_w.shape[0]
     n = n_all - extra
+    _need(group_mark in MOE_GROUP_MARKS, f"group_mark {group_mark!r}: one of {tuple(MOE_GROUP_MARKS)}")
     _need(scoring in MOE_SCORINGS and 0 <= extra < n_all, f"scoring {scoring!r} (one of {sorted(MOE_SCORINGS)}), {extra} extra rows of {n_all}")
     _need(router_w.dtype == torch.float32 and router_w.shape == (n_all, W) and router_w.is_contiguous(), f"router: float32 [n, {W}]")
     _need(correction is None or (correction.dtype == torch.float32 and correction.shape == (n,) and correction.is_contiguous()), f"correction: float32 [{n}]")
@@ -2102,8 +2151,8 @@ def moe_route(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor 
     weights = torch.empty((T, top), dtype=torch.float32, device=h.device)
     extras = torch.empty((T, extra), dtype=torch.float32, device=h.device) if extra else None
     _check(_fn("moe.hip", "pllm_moe_route", signature=[c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                                        c_int, c_void_p, c_void_p, c_void_p, c_void_p])(
-        dtype_code(h.dtype), _ptr(h), h.stride(0), _ptr(router_w), _ptr(correction), T, W, n_all, extra, MOE_SCORINGS[scoring], groups, keep, top,
+                                                        c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p])(
+        dtype_code(h.dtype), _ptr(h), h.stride(0), _ptr(router_w), _ptr(correction), T, W, n_all, extra, MOE_SCORINGS[scoring], groups, keep, MOE_GROUP_MARKS[group_mark], top,
         _ptr(ids), _ptr(weights), _ptr(extras), _stream()), "moe_route")
     return (ids, weights, extras) if extra else (ids, weights)
 

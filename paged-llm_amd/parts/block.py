@@ -86,7 +86,10 @@ class BranchNormBlock(Block):
         a = p["mixer"].forward(self._rows(x, ctx), ctx, cache, state)
         self._add(p["mixer_norm"], x, a, ctx)
         if self.has_feed_forward:
+            # a feed-forward may hand over a sum that the norm's kernel forms (``ops.ChoiceSum``)
+            ctx.branch_sum_ok = bool(getattr(p["feed_forward_norm"], "takes_choice_sum", False))
             m = p["feed_forward"].forward(self._rows(x, ctx), ctx)
+            ctx.branch_sum_ok = False
             self._add(p["feed_forward_norm"], x, m, ctx)
         ctx.float_branch = False
         return x, None

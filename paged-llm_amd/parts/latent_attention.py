@@ -14,7 +14,8 @@ windowed group.
 
 Options that a layer may have: no rotated part at all (``rot_dim`` 0: no positions enter the scores), queries that come
 through a latent of their own (``q_rank``: c_q = RMS norm of W_dq h with a weight, the heads' queries W_uq c_q), and a gate
-per head on the attention's output (``head_gate``: head h's values times sigmoid((W_g h)_h)).
+per head on the attention's output (``head_gate``: head h's values times sigmoid((W_g h)_h)), and a learned logit per head that
+takes part in the softmax's sum and in nothing else (``sinks``).
 """
 
 from __future__ import annotations
@@ -32,10 +33,10 @@ from .spec import PartSpec, WeightSpec
 class LatentAttention(Mixer):
     """params: ``heads``, ``plain_dim``, ``rot_dim`` (per head; 0: none), ``head_dim`` (of the values), ``rank``, ``scale``,
     ``window`` (0: none), ``position`` (the rotary spec of the rot part; None without one), ``eps`` (of the latents' norms),
-    ``q_rank`` (0: queries straight from the input; only without a rotated part), ``head_gate``.
+    ``q_rank`` (0: queries straight from the input; only without a rotated part), ``head_gate``, ``sinks``.
     Tensors ``q`` [heads (plain + rot), width] or, with ``q_rank``, ``dq`` [q_rank, width], ``dq.norm`` [q_rank] and ``uq``
     [heads plain, q_rank]; ``dkv`` [rank + rot, width], ``dkv.norm`` [rank], ``uk`` [heads plain, rank], ``uv`` [heads
-    head_dim, rank], ``o`` [width, heads head_dim]; ``g`` [heads, width] with ``head_gate``."""
+    head_dim, rank], ``o`` [width, heads head_dim]; ``g`` [heads, width] with ``head_gate``; ``sink`` [heads] with ``sinks``."""
     graph_capturable = True
     graph_capturable_prompts = True
 
@@ -45,6 +46,7 @@ class LatentAttention(Mixer):
         self.P, self.rank = int(params["head_dim"]), int(params["rank"])
         self.scale, self.window, self.eps = float(params["scale"]), int(params.get("window") or 0), float(params["eps"])
         self.q_rank, self.head_gate = int(params.get("q_rank") or 0), bool(params.get("head_gate"))
+        self.has_sinks = bool(params.get("sinks"))
         if self.rank > ops.MAX_LATENT_RANK or self.rot > ops.MAX_LATENT_ROT or self.rot % 2 or self.rot < 0 or self.plain <= 0:
             raise ValueError(f"latent attention takes a rank up to {ops.MAX_LATENT_RANK}, an even rotated width up to "
                              f"{ops.MAX_LATENT_ROT} and a plain width of at least 1; got {self.rank}, {self.rot}, {self.plain}")
@@ -60,7 +62,7 @@ class LatentAttention(Mixer):
         self.width = -(-(self.rank + self.rot) // 16) * 16            # of a key row in the pages
         self.paged = self.width <= ops.MAX_HEAD_DIM_GENERIC           # the paged attention kernels take it
         self._w: dict = {}
-        self.w_in = self.w_o = self.w_uk_t = self.w_uv = self.norm_w = self.w_uq = self.q_norm_w = self.w_g = None
+        self.w_in = self.w_o = self.w_uk_t = self.w_uv = self.norm_w = self.w_uq = self.q_norm_w = self.w_g = self.sinks = self.terms = None
 
     def weight_specs(self):
         H = self.heads
@@ -74,6 +76,8 @@ class LatentAttention(Mixer):
             specs["q"] = WeightSpec((H * (self.plain + self.rot), self.hidden))
         if self.head_gate:
             specs["g"] = WeightSpec((H, self.hidden))
+        if self.has_sinks:
+            specs["sink"] = WeightSpec((H,), role="vector")
         return specs
 
     def assign(self, name, tensor):
@@ -92,9 +96,12 @@ class LatentAttention(Mixer):
             self.w_in = Weight(torch.cat([w.pop("q"), w.pop("dkv")], dim=0).contiguous())
             self.w_g = Weight(w.pop("g")) if self.head_gate else None
         self.w_o = Weight(w.pop("o"))
-        self.w_uk_t = w.pop("uk").view(H, self.plain, self.rank).transpose(1, 2).contiguous()     # [heads, rank, plain]: qa = W_uk^T q
-        self.w_uv = w.pop("uv").view(H, self.P, self.rank).contiguous()
+        self.w_uk_t = ops.HeadMatrices(w.pop("uk").view(H, self.plain, self.rank).transpose(1, 2))     # per head [rank, plain]: qa = W_uk^T q
+        self.w_uv = ops.HeadMatrices(w.pop("uv").view(H, self.P, self.rank))
         self.norm_w = w.pop("dkv.norm")
+        if self.has_sinks:
+            self.sinks = w.pop("sink")
+            self.terms = ops.ScoreTerms(0.0, None, self.sinks)
 
     def cache_spec(self):
         kind = "window" if self.window > 0 else "full"
@@ -138,9 +145,10 @@ class LatentAttention(Mixer):
         ops.gemm_heads(q_plain, self.w_uk_t, out=q[:, :, :rank])
         if self.paged:
             mixed = ops.paged_attention(q.view(T, H * width), k_pages, v_pages, view.block_tables, ctx.cu_seqlens_q, ctx.seq_lens_k,
-                                        H, 1, width, self.scale, self.window, ctx).view(T, H, width)[:, :, :rank]
+                                        H, 1, width, self.scale, self.window, ctx, terms=self.terms).view(T, H, width)[:, :, :rank]
         else:
-            mixed = ops.latent_attention(q, rank, r, k_pages, view.block_tables, ctx.cu_seqlens_q, ctx.seq_lens_k, self.scale, self.window)
+            mixed = ops.latent_attention(q, rank, r, k_pages, view.block_tables, ctx.cu_seqlens_q, ctx.seq_lens_k, self.scale, self.window,
+                                         self.sinks)
         values = ops.gemm_heads(mixed, self.w_uv).view(T, H * self.P)
         if gate is not None:
             values = ops.gate_heads(values, gate, H, self.P, self.P)

@@ -4,7 +4,7 @@ router scores as weights.
 
 Router: z = W_router h in float, scores s = softmax(z) over all router outputs.  The choice looks at s + correction (a
 stored vector): the experts are cut into ``groups`` equal groups of neighbours, a group's mark is its largest corrected
-score, and only experts of the ``keep`` best groups can be chosen; the ``top`` largest corrected scores among those win.
+score (or the sum of its two largest: ``group_mark`` "two_largest"), and only experts of the ``keep`` best groups can be chosen; the ``top`` largest corrected scores among those win.
 The weights are the chosen experts' scores s themselves (no renormalisation).  The last ``identity`` router outputs
 stand for experts without weights that hand the token's own row back.
 
@@ -33,7 +33,7 @@ from .spec import WeightSpec
 
 class RoutedExperts(FeedForward):
     """params: ``experts``, ``identity`` (pass-through experts behind them, default 0), ``top``, ``groups`` and ``keep``
-    (defaults 1 and 1), ``intermediate_size`` (of one expert), ``activation`` (default "silu"), ``correction`` (a stored
+    (defaults 1 and 1), ``group_mark`` ("largest" or "two_largest"), ``intermediate_size`` (of one expert), ``activation`` (default "silu"), ``correction`` (a stored
     vector is added to the scores for the choice; default True), ``scoring`` ("softmax" or "sigmoid"), ``weight_on``
     ("output" or "input"), ``gated`` (default True; False: experts without a gate matrix, whose activation is one of
     ``ops.ROW_ACTIVATIONS`` without parameters), ``router_bias`` (the name of a stored vector added to the router's outputs; with
@@ -48,6 +48,7 @@ class RoutedExperts(FeedForward):
         self.experts, self.identity = int(params["experts"]), int(params.get("identity") or 0)
         self.top, self.groups, self.keep = int(params["top"]), int(params.get("groups") or 1), int(params.get("keep") or 1)
         self.inter = int(params["intermediate_size"])
+        self.group_mark = params.get("group_mark", "largest")
         self.activation = params.get("activation", "silu")
         self.has_correction = bool(params.get("correction", True))
         self.scoring, self.weight_on = params.get("scoring", "softmax"), params.get("weight_on", "output")
@@ -55,6 +56,8 @@ class RoutedExperts(FeedForward):
         shared = params.get("shared") or None
         self.shared_inter = int(shared["intermediate_size"]) if shared else 0
         self.shared_gate = bool(shared.get("gate", False)) if shared else False
+        if self.group_mark not in ops.MOE_GROUP_MARKS:
+            raise ValueError(f"group_mark {self.group_mark!r}: one of {tuple(ops.MOE_GROUP_MARKS)}")
         if self.scoring not in ops.MOE_SCORINGS or self.weight_on not in ("output", "input"):
             raise ValueError(f"scoring {self.scoring!r} (one of {sorted(ops.MOE_SCORINGS)}), weight_on {self.weight_on!r} (output or input)")
         self.n = self.experts + self.identity
@@ -112,7 +115,8 @@ class RoutedExperts(FeedForward):
     def forward(self, h, ctx):
         h = rows_of(h)
         inside = self.weight_on == "input"
-        routed = ops.moe_route(h, self.router, self.correction, self.groups, self.keep, self.top, self.scoring, extra=1 if self.shared_gate else 0)
+        routed = ops.moe_route(h, self.router, self.correction, self.groups, self.keep, self.top, self.scoring, extra=1 if self.shared_gate else 0,
+                               group_mark=self.group_mark)
         ids, weights = routed[0], routed[1]
         rows = ops.moe_tile_rows(ids.numel(), self.experts, h.dtype, self.hidden, self.inter, h.stride(0))
         sorted_pair, row_of_pair, tiles = ops.moe_align(ids, self.experts, rows)

@@ -162,13 +162,17 @@ class LayerNorm(Norm):
     kernel (a block that norms what its branches return, not what they read).
 
     params: ``eps``; ``size`` (default: the model's width); ``weight_name`` / ``bias_name``: the tensors' own names
-    under the part's prefix (defaults "weight" and "bias"; "" is the prefix itself)."""
+    under the part's prefix (defaults "weight" and "bias"; "" is the prefix itself); ``factor``: a constant by which weight and
+    bias are multiplied in float when they arrive, y times the constant (a scale of the logits, which are linear in the last
+    norm's rows, costs nothing there)."""
+    takes_choice_sum = True             # ``add_to`` forms a branch that is a sum of experts' rows (``ops.ChoiceSum``) in its kernel
 
     def __init__(self, params: dict, env: BuildEnv):
         self.eps = float(params["eps"])
         self.size = int(params.get("size", env.hidden_size))
         self.weight_name = params.get("weight_name", "weight")
         self.bias_name = params.get("bias_name", "bias")
+        self.factor = float(params.get("factor", 1.0))
         self.dtype, self.device = env.dtype, env.device
         self.weight: torch.Tensor | None = None
         self.bias: torch.Tensor | None = None
@@ -179,6 +183,8 @@ class LayerNorm(Norm):
 
     def assign(self, name, tensor):
         t = tensor.to(device=self.device, dtype=torch.float32).contiguous()
+        if self.factor != 1.0:
+            t = t * self.factor
         if name == self.weight_name:
             self.weight = t
         elif name == self.bias_name:
@@ -190,8 +196,8 @@ class LayerNorm(Norm):
         """The normed rows in the compute type (x: float or compute-type rows)."""
         return ops.layernorm(x, self.weight, self.bias, self.eps, None, row_index, self.dtype)
 
-    def add_to(self, stream: torch.Tensor, branch: torch.Tensor, want_rows: bool = True):
-        """stream += norm(branch), in place and in float; returns the new stream rounded to the compute type when that
+    def add_to(self, stream: torch.Tensor, branch, want_rows: bool = True):
+        """stream += norm(branch), in place and in float (the branch rows, or an ``ops.ChoiceSum``); returns the new stream rounded to the compute type when that
         is another type than the stream's and ``want_rows`` (the next product's operand), else None."""
         out_dtype = self.dtype if want_rows and self.dtype != stream.dtype else None
         return ops.layernorm(branch, self.weight, self.bias, self.eps, stream, None, out_dtype)

@@ -3,7 +3,8 @@ pages: usually divided by their root mean square per head (``qk_norm``; a layer 
 
 q, k, v (and one gate per head) from one product of the mixer's input -> optional biases -> optional short causal
 convolution over time on every channel of q, k and v (the last taps - 1 projected rows of a request are its state) ->
-rotary encoding of q and k -> q and k of every head divided by their root mean square (an RMS norm without a weight) ->
+rotary encoding of q and k -> q and k of every head divided by their root mean square (an RMS norm, without a weight or with
+one that all heads share; it may stand in front of the rotation instead) ->
 k and v into their pages -> attention with a causal mask that is full, a sliding window, or blocks of positions counted
 from position 0 (a query sees the keys of its own block only), optionally with a learned logit per head in the softmax's
 denominator -> optionally every head's output times the sigmoid of its gate -> output product, optionally with a bias.
@@ -32,7 +33,8 @@ class NormedAttention(Mixer):
     rotary spec or None), ``mask`` ("full", "window" or "chunk") with ``mask_size``, ``conv`` (taps of the convolution
     over time; 0: none), ``bias`` (q, k, v and the output product have biases), ``sinks`` (a logit per head in the
     softmax's sum), ``head_gate`` (a gate per head from the mixer's input), ``qk_norm`` (default True; False: q and k go
-    to the scores as they are rotated), ``score_cap`` c > 0 (the scaled product x becomes c tanh(x / c); default none);
+    to the scores as they are rotated), ``norm_weights`` (that norm has a weight for q and one for k, [key_dim] each, shared by the heads),
+    ``norm_first`` (the norm stands in front of the rotation), ``score_cap`` c > 0 (the scaled product x becomes c tanh(x / c); default none);
     ``output_bias`` (default: as ``bias``; False: the projections have biases, the output product has none);
     ``values``: "projected" (default), "normed" (every value head divided by its root mean square, ``eps`` inside the root, no
     weight, and cached so) or "keys" (there is no value product: a value head is its key head as projected, before the
@@ -40,7 +42,7 @@ class NormedAttention(Mixer):
     still sees, at their own positions); ``weighting``: "softmax" (default) or "sigmoid" (a visible key weighs
     sigmoid(score + ``pb``[head]), not normalised over the keys).  Tensors (under the part's prefix): ``q``,
     ``k``, ``v``, ``o``; ``q.b``, ``k.b``, ``v.b``, ``o.b``; ``q.conv``, ``k.conv``, ``v.conv`` [channels, taps];
-    ``sink`` [heads]; ``g`` [heads, width]; ``pb`` [heads]."""
+    ``sink`` [heads]; ``g`` [heads, width]; ``pb`` [heads]; ``q.norm``, ``k.norm`` [key_dim]."""
     graph_capturable = True
     graph_capturable_prompts = True
 
@@ -54,6 +56,7 @@ class NormedAttention(Mixer):
         self.taps = max(1, int(params.get("conv") or 1))
         self.bias, self.has_sinks, self.head_gate = bool(params.get("bias")), bool(params.get("sinks")), bool(params.get("head_gate"))
         self.qk_norm, self.score_cap = bool(params.get("qk_norm", True)), float(params.get("score_cap") or 0.0)
+        self.norm_first, self.has_norm_weights = bool(params.get("norm_first")), bool(params.get("norm_weights"))
         self.out_bias = bool(params.get("output_bias", self.bias))
         self.values = params.get("values") or "projected"
         self.keep_first = int(params.get("keep_first") or 0)
@@ -66,6 +69,8 @@ class NormedAttention(Mixer):
             raise ValueError("first positions are kept beside a sliding window only")
         if self.weighting == "sigmoid" and self.has_sinks:
             raise ValueError("a sink is a term of a softmax's sum: there is none under sigmoid weights")
+        if self.has_norm_weights and not self.qk_norm:
+            raise ValueError("weights of the q/k norm belong to a q/k norm")
         if self.score_cap < 0.0:
             raise ValueError(f"a cap of the scores is positive (or 0 for none), got {self.score_cap}")
         if self.heads % self.kv_heads:
@@ -85,7 +90,7 @@ class NormedAttention(Mixer):
         # the mask as the attention kernels take it: > 0 a window, < 0 blocks of that many positions
         self.window = self.mask_size if self.mask == "window" else (-self.mask_size if self.mask == "chunk" else 0)
         self._w: dict = {}
-        self.w_in = self.w_o = self.b_in = self.output_bias = self.conv_w = self.terms = self.weights = None
+        self.w_in = self.w_o = self.b_in = self.output_bias = self.conv_w = self.terms = self.weights = self.norm_w = None
 
     # ---- weights
     def weight_specs(self):
@@ -104,6 +109,8 @@ class NormedAttention(Mixer):
             specs.update({f"{n}.conv": WeightSpec((c, self.taps), role="vector") for n, c in (("q", q), ("k", k), ("v", v))[:3 if own_values else 2]})
         if self.weighting == "sigmoid":
             specs["pb"] = WeightSpec((self.heads,), role="vector")
+        if self.has_norm_weights:
+            specs.update({n: WeightSpec((self.d,), role="vector", init="ones") for n in ("q.norm", "k.norm")})
         if self.has_sinks:
             specs["sink"] = WeightSpec((self.heads,), role="vector")
         if self.head_gate:
@@ -127,6 +134,8 @@ class NormedAttention(Mixer):
             self.output_bias = w.pop("o.b")           # added by whoever norms the mixer's float output (the block's kernel), or by the product
         if self.has_conv:
             self.conv_w = torch.cat([w.pop(n + ".conv") for n in qkv], dim=0).contiguous()
+        if self.has_norm_weights:
+            self.norm_w = (w.pop("q.norm"), w.pop("k.norm"))
         if self.keep_first or self.weighting == "sigmoid":
             self.weights = ops.KeyWeights(self.keep_first, self.weighting == "sigmoid", w.pop("pb") if self.weighting == "sigmoid" else None)
         terms = ops.ScoreTerms(self.score_cap, None, w.pop("sink") if self.has_sinks else None)
@@ -158,7 +167,8 @@ class NormedAttention(Mixer):
         q = ops.attn_prepare(proj, self.b_in, self.conv_w, state, ctx.state_slots, ctx.seq_starts, ctx.cu_seqlens_q, ctx.num_seqs,
                              ctx.positions, pe.cos if pe is not None else None, pe.sin if pe is not None else None, self.rot,
                              bool(pe.interleaved) if pe is not None else False, self.eps, H, G, self.d, self.dv, D, self.dtype,
-                             view.slot_mapping, k_pages, v_pages, qk_norm=self.qk_norm, values=self.values)
+                             view.slot_mapping, k_pages, v_pages, qk_norm=self.qk_norm, values=self.values,
+                             norm_weights=self.norm_w, norm_first=self.norm_first)
         o = ops.paged_attention(q, k_pages, v_pages, view.block_tables, ctx.cu_seqlens_q, ctx.seq_lens_k, H, G, D, self.scale,
                                 self.window, ctx, terms=self.terms, weights=self.weights)
         if self.head_gate or D != self.dv:
