@@ -45,6 +45,31 @@ MODELS = {
 }
 
 
+def measure_models(models: dict, width: int, dtype: str, context: int, steps: int, warmup: int) -> dict:
+    """{name_w<width>: numbers} of every configuration (random weights), one engine at a time: prefill (one prompt of 512 and of
+    2048 tokens in one step) and decode (1, 8 and 64 requests at ``context``)."""
+    import torch
+    out = {}
+    for name, cfg in models.items():
+        row = {}
+        with tempfile.TemporaryDirectory() as folder:
+            engine = make_engine(cfg, folder, dtype, 64, context)
+            for tokens in (512, PREFILL_TOKENS):
+                t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
+                row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
+                row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
+            for batch in (1, 8, 64):
+                sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
+                row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
+                row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
+            row["weights_millions"] = round(sum(_weights_of(engine.model)) / 1e6, 1)
+            del engine
+            torch.cuda.empty_cache()
+        out[f"{name}_w{width}"] = row
+        print(f"[bench] {name} width {width}: {row}", file=sys.stderr, flush=True)
+    return out
+
+
 def gudutar_config(width: int, periods: int, vocab: int, window: int = 1024) -> dict:
     """Gudutar at sizes that resemble a real model's layers: ``periods`` times [state-space, state-space, retention,
     latent attention with a feed-forward].  State-space layers of twice the width in heads of 64 channels with 128 state
@@ -69,7 +94,6 @@ def run_gudutar(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
     the Llama decoder at the same width, number of layers, feed-forward width and vocabulary (random weights).  The
     Llama model has a feed-forward on every layer and Gudutar on every fourth, so the pairs differ in weight; what is
     compared is tokens per second and, per mixer, what its kernels take (see the profiles)."""
-    import torch
     out = {}
     for width in widths:
         periods = 3
@@ -78,23 +102,7 @@ def run_gudutar(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
             "llama": dict(TINYLLAMA, num_hidden_layers=4 * periods, hidden_size=width, num_attention_heads=width // 64,
                           num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
         }
-        for name, cfg in models.items():
-            row = {}
-            with tempfile.TemporaryDirectory() as folder:
-                engine = make_engine(cfg, folder, dtype, 64, context)
-                for tokens in (512, PREFILL_TOKENS):
-                    t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
-                    row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
-                    row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
-                for batch in (1, 8, 64):
-                    sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
-                    row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
-                    row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
-                params = sum(_weights_of(engine.model))
-                row["weights_millions"] = round(params / 1e6, 1)
-                del engine
-                torch.cuda.empty_cache()
-            out[f"{name}_w{width}"] = row
+        out.update(measure_models(models, width, dtype, context, steps, warmup))
     return out
 
 
@@ -121,7 +129,6 @@ def run_mutapel(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
     Mutapel beside the Llama decoder at the same width, number of layer runs, heads, active feed-forward width and
     vocabulary (random weights).  Mutapel holds 30 experts where the Llama model holds one feed-forward, so it is far
     heavier in weights; per token it multiplies by as many."""
-    import torch
     out = {}
     for width in widths:
         models = {
@@ -129,22 +136,7 @@ def run_mutapel(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
             "llama": dict(TINYLLAMA, num_hidden_layers=12, hidden_size=width, num_attention_heads=width // 64,
                           num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
         }
-        for name, cfg in models.items():
-            row = {}
-            with tempfile.TemporaryDirectory() as folder:
-                engine = make_engine(cfg, folder, dtype, 64, context)
-                for tokens in (512, PREFILL_TOKENS):
-                    t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
-                    row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
-                    row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
-                for batch in (1, 8, 64):
-                    sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
-                    row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
-                    row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
-                row["weights_millions"] = round(sum(_weights_of(engine.model)) / 1e6, 1)
-                del engine
-                torch.cuda.empty_cache()
-            out[f"{name}_w{width}"] = row
+        out.update(measure_models(models, width, dtype, context, steps, warmup))
     return out
 
 
@@ -173,7 +165,6 @@ def run_nesezen(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
     """Prefill (one prompt of 512 and of 2048 tokens in one step) and decode (1, 8 and 64 requests at ``context``) of
     Nesezen beside the two closest decoders at the same width, twelve layers and vocabulary (random weights): Gudutar (a
     float residual stream, recurrent layers with a state per request, latent attention) and the Llama decoder."""
-    import torch
     out = {}
     for width in widths:
         models = {
@@ -182,23 +173,7 @@ def run_nesezen(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
             "llama": dict(TINYLLAMA, num_hidden_layers=12, hidden_size=width, num_attention_heads=width // 64,
                           num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
         }
-        for name, cfg in models.items():
-            row = {}
-            with tempfile.TemporaryDirectory() as folder:
-                engine = make_engine(cfg, folder, dtype, 64, context)
-                for tokens in (512, PREFILL_TOKENS):
-                    t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
-                    row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
-                    row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
-                for batch in (1, 8, 64):
-                    sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
-                    row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
-                    row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
-                row["weights_millions"] = round(sum(_weights_of(engine.model)) / 1e6, 1)
-                del engine
-                torch.cuda.empty_cache()
-            out[f"{name}_w{width}"] = row
-            print(f"[bench] {name} width {width}: {row}", file=sys.stderr, flush=True)
+        out.update(measure_models(models, width, dtype, context, steps, warmup))
     return out
 
 
@@ -232,7 +207,6 @@ def run_renadra(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
     Renadra beside the two closest decoders at the same width, twelve layer runs and vocabulary (random weights): Nesezen (a
     pre-norm block over a float residual stream, windowed attention with capped scores, a recurrence with a state per
     request) and the Llama decoder."""
-    import torch
     out = {}
     for width in widths:
         models = {
@@ -241,23 +215,7 @@ def run_renadra(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
             "llama": dict(TINYLLAMA, num_hidden_layers=12, hidden_size=width, num_attention_heads=width // 64,
                           num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
         }
-        for name, cfg in models.items():
-            row = {}
-            with tempfile.TemporaryDirectory() as folder:
-                engine = make_engine(cfg, folder, dtype, 64, context)
-                for tokens in (512, PREFILL_TOKENS):
-                    t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
-                    row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
-                    row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
-                for batch in (1, 8, 64):
-                    sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
-                    row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
-                    row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
-                row["weights_millions"] = round(sum(_weights_of(engine.model)) / 1e6, 1)
-                del engine
-                torch.cuda.empty_cache()
-            out[f"{name}_w{width}"] = row
-            print(f"[bench] {name} width {width}: {row}", file=sys.stderr, flush=True)
+        out.update(measure_models(models, width, dtype, context, steps, warmup))
     return out
 
 
@@ -283,7 +241,6 @@ def run_mekusun(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
     Mekusun beside the closest decoders at the same width, twelve layers and vocabulary (random weights): Nesezen (a matrix
     memory, latent attention, routed experts), Gudutar (a state-space layer with a convolution, latent attention with a
     rotated part, norms behind the branches) and the Llama decoder."""
-    import torch
     out = {}
     for width in widths:
         models = {
@@ -293,23 +250,42 @@ def run_mekusun(dtype: str, context: int, steps: int, warmup: int, widths=(1024,
             "llama": dict(TINYLLAMA, num_hidden_layers=12, hidden_size=width, num_attention_heads=width // 64,
                           num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
         }
-        for name, cfg in models.items():
-            row = {}
-            with tempfile.TemporaryDirectory() as folder:
-                engine = make_engine(cfg, folder, dtype, 64, context)
-                for tokens in (512, PREFILL_TOKENS):
-                    t = time_prefill(engine, tokens, seed=100 + tokens, repeats=4)
-                    row[f"prefill_{tokens}_ms"] = round(t * 1e3, 3)
-                    row[f"prefill_{tokens}_tok_per_s"] = round(tokens / t, 1)
-                for batch in (1, 8, 64):
-                    sec, _ = time_decode(engine, batch, context, steps, warmup, seed=batch)
-                    row[f"decode_b{batch}_ms"] = round(sec * 1e3, 4)
-                    row[f"decode_b{batch}_tok_per_s"] = round(batch / sec, 1)
-                row["weights_millions"] = round(sum(_weights_of(engine.model)) / 1e6, 1)
-                del engine
-                torch.cuda.empty_cache()
-            out[f"{name}_w{width}"] = row
-            print(f"[bench] {name} width {width}: {row}", file=sys.stderr, flush=True)
+        out.update(measure_models(models, width, dtype, context, steps, warmup))
+    return out
+
+
+def pamunex_config(width: int, vocab: int, window: int = 1024, block: int = 2048) -> dict:
+    """Pamunex at sizes that resemble a real model's layers: six periods of [latent attention + dense feed-forward, attention over
+    blocks + routed experts].  Sixteen latent heads of 128 elements and a rotated part of 64 over a latent of 192, a window of
+    ``window`` positions; grouped heads of 64 as the Llama model beside it has, one key head per eight heads, blocks of ``block``
+    positions; dense feed-forwards of four times the width (no gate: two matrices); 16 experts as wide as the model of which 4 are
+    chosen (4 groups of 4, the best 2 kept), so the chosen ones do the work of the dense feed-forward."""
+    heads = width // 64
+    lat = {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 192, "rot_dim": 64, "rot": {"base": 10000.0, "dims": 64}, "scale": (128 + 64) ** -0.5,
+           "mask": {"size": window}}
+    att = {"heads": heads, "kv_heads": max(1, heads // 8), "dim": 64, "vdim": 64, "rot": {"base": 10000.0, "dims": 64}, "scale": 0.125, "mask": {"size": block}}
+    moe = {"kind": "moe", "expert": {"ff": width}, "router": {"experts": 16, "top": 4, "groups": {"count": 4, "keep": 2}}}
+    period = [{"type": "latent_attention", "mixer": lat, "mlp": {"kind": "dense", "ff": 4 * width}}, {"type": "attention", "mixer": att, "mlp": moe}]
+    return {"architecture": "Pamunex", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_scale": 0.5,
+            "layers": [dict(l) for _ in range(6) for l in period], "max_positions": 4096, "torch_dtype": "bfloat16"}
+
+
+def run_pamunex(dtype: str, context: int, steps: int, warmup: int, widths=(1024, 2048)) -> dict:
+    """Prefill (one prompt of 512 and of 2048 tokens in one step) and decode (1, 8 and 64 requests at ``context``) of
+    Pamunex beside the closest decoders at the same width, twelve layers (or layer runs) and vocabulary (random weights): Mutapel
+    (attention over blocks with a sink, experts in groups), Gudutar (latent attention under a window, layer norms behind the
+    branches), Mekusun (ungated feed-forwards and experts) and the Llama decoder."""
+    out = {}
+    for width in widths:
+        models = {
+            "pamunex": pamunex_config(width, 32000),
+            "mutapel": mutapel_config(width, 32000),
+            "gudutar": gudutar_config(width, 3, 32000),
+            "mekusun": mekusun_config(width, 32000),
+            "llama": dict(TINYLLAMA, num_hidden_layers=12, hidden_size=width, num_attention_heads=width // 64,
+                          num_key_value_heads=max(1, width // 512), head_dim=64, intermediate_size=11 * width // 4, torch_dtype=dtype),
+        }
+        out.update(measure_models(models, width, dtype, context, steps, warmup))
     return out
 
 
@@ -843,7 +819,9 @@ def main() -> int:
                     "attention, windowed attention with normed values, gated recurrences, a bigram embedding, repeated layers) beside Nesezen and the Llama decoder at equal sizes, instead")
     ap.add_argument("--mekusun", action="store_true", help="prefill and decode of the Mekusun decoder (a selective scan, a delta memory, latent attention, "
                     "ungated experts, a weighted sum over the depth) beside Nesezen, Gudutar and the Llama decoder at equal sizes, instead")
-    ap.add_argument("--widths", default=None, metavar="N,N", help="model widths of --renadra and --mekusun (default 1024,2048)")
+    ap.add_argument("--pamunex", action="store_true", help="prefill and decode of the Pamunex decoder (latent attention under a window, attention over blocks, "
+                    "sinks, ungated feed-forwards and experts) beside Mutapel, Gudutar, Mekusun and the Llama decoder at equal sizes, instead")
+    ap.add_argument("--widths", default=None, metavar="N,N", help="model widths of --renadra, --mekusun and --pamunex (default 1024,2048)")
     ap.add_argument("--kernels", action="store_true", help="every kernel of a decode step and of a prompt step on its own, with its fraction")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -887,6 +865,12 @@ def main() -> int:
         print(json.dumps({"metric": "Mekusun beside Nesezen, Gudutar and the Llama decoder at equal width, depth and vocabulary (random weights): prefill and decode",
                           "dtype": short, "context": args.context,
                           "models": run_mekusun(args.dtype, args.context, max(16, args.steps // 2), max(4, args.warmup // 2), widths)}))
+        return 0
+    if args.pamunex:
+        widths = tuple(int(w) for w in args.widths.split(",")) if args.widths else (1024, 2048)
+        print(json.dumps({"metric": "Pamunex beside Mutapel, Gudutar, Mekusun and the Llama decoder at equal width, layer runs and vocabulary (random weights): prefill and decode",
+                          "dtype": short, "context": args.context,
+                          "models": run_pamunex(args.dtype, args.context, max(16, args.steps // 2), max(4, args.warmup // 2), widths)}))
         return 0
     if args.workload == "ragged64":
         print(json.dumps({"metric": f"output tokens/s, 64 ragged requests at once, prompts 64-2048 tokens, 256 generated each ({model_name}, random weights)",

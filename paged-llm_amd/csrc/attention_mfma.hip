@@ -31,12 +31,15 @@ using namespace pllm;
 static_assert(HEAD_DIM % 16 == 0 && HEAD_DIM >= 16 && HEAD_DIM <= 256, "head size must be 16..256 in steps of 16");
 
 // -DSCORE_TERMS=1 compiles the kernels with the further terms of a score (a cap, a slope times the distance, a sink
-// per head: ScoreTerms in common.h) as one more argument.  Without it there is no such argument: `terms` then names a
+// per head: ScoreTerms in common.h) as one more argument; -DSCORE_TERMS=2 with the sinks alone, which change where a column's
+// softmax starts and nothing in the loops (the other terms' code there costs a quarter of the prompt kernel's time at
+// head size 256 even where none of them is given).  Without it there is no such argument: `terms` then names a
 // constant that says "none", and everything that reads it is compiled out.
 #ifndef SCORE_TERMS
 #define SCORE_TERMS 0
 #endif
-constexpr bool kTerms = SCORE_TERMS != 0;
+static_assert(SCORE_TERMS >= 0 && SCORE_TERMS <= 2, "0: no further terms, 1: all, 2: sinks alone");
+constexpr bool kTerms = SCORE_TERMS != 0, kForms = SCORE_TERMS == 1;      // kForms: scores are brought to another form in the loops
 #if SCORE_TERMS
 #define PLLM_TERMS_PARAM , ScoreTerms terms
 #define PLLM_TERMS_ARG , terms
@@ -204,7 +207,7 @@ __global__ __launch_bounds__(WAVES * 64) void paged_attention_mfma_kernel(
     const size_t row = (size_t)(q_begin + tok) * q_stride + (size_t)(kvh * G + hg) * D;
     my_out[cb] = (size_t)(q_begin + tok) * out_stride + (size_t)(kvh * G + hg) * D;
     if constexpr (kTerms) {
-      my_slope[cb] = (terms.slopes && my_valid[cb]) ? terms.slopes[kvh * G + hg] * kLog2e : 0.f;
+      my_slope[cb] = (kForms && terms.slopes && my_valid[cb]) ? terms.slopes[kvh * G + hg] * kLog2e : 0.f;
       my_sink[cb] = (terms.sinks && my_valid[cb]) ? terms.sinks[kvh * G + hg] * kLog2e : -INFINITY;
     }
 #pragma unroll
@@ -308,7 +311,7 @@ __global__ __launch_bounds__(WAVES * 64) void paged_attention_mfma_kernel(
       float sc[4][4];
       float mx = -INFINITY;
       float mul = sl2;
-      if constexpr (kTerms) {
+      if constexpr (kForms) {
         if (form.any()) {
           float s[4][4];
 #pragma unroll
@@ -609,7 +612,7 @@ __global__ __launch_bounds__(256 * KG, (D <= 96 || KG == 2) ? 2 : 1) void paged_
     const size_t row = (size_t)(q_begin + tok) * q_stride + (size_t)(kvh * G + hg) * D;
     my_out[cb] = (size_t)(q_begin + tok) * out_stride + (size_t)(kvh * G + hg) * D;
     if constexpr (kTerms) {
-      my_slope[cb] = (terms.slopes && my_valid[cb]) ? terms.slopes[kvh * G + hg] * kLog2e : 0.f;
+      my_slope[cb] = (kForms && terms.slopes && my_valid[cb]) ? terms.slopes[kvh * G + hg] * kLog2e : 0.f;
       my_sink[cb] = (terms.sinks && my_valid[cb]) ? terms.sinks[kvh * G + hg] * kLog2e : -INFINITY;
     }
 #pragma unroll
@@ -762,7 +765,7 @@ __global__ __launch_bounds__(256 * KG, (D <= 96 || KG == 2) ? 2 : 1) void paged_
       // maximum m_run is kept in scaled log2 units.  (With further terms the scores are brought to their final
       // form in log2 units first, and the factor below is one.)
       float mul = sl2;
-      if constexpr (kTerms) {
+      if constexpr (kForms) {
         if (form.any()) {
           float s[4][4];
 #pragma unroll
@@ -1202,8 +1205,8 @@ PLLM_API int pllm_paged_attention_mfma(const void* q, int q_stride, const void* 
 // The same with a hint for the prompt kernel's form (single_prompt: all queries but a few belong to one sequence) and
 // with further terms of the score: score_cap > 0 caps the scaled products (c tanh(x / c)), slopes [heads]
 // adds slope * (key position - query position), sinks [heads] gives every head a logit that takes part in the
-// softmax's sum only (null: none).  A library compiled without -DSCORE_TERMS=1 refuses any of them.
-PLLM_API int pllm_attention_mfma_score_terms() { return kTerms ? 1 : 0; }
+// softmax's sum only (null: none).  A library refuses the terms it was compiled without.
+PLLM_API int pllm_attention_mfma_score_terms() { return SCORE_TERMS; }
 
 PLLM_API int pllm_paged_attention_mfma_terms(const void* q, int q_stride, const void* k_pages, const void* v_pages, void* out,
                                              int out_stride, const int* block_tables, int bt_stride, const int* cu_seqlens_q,
@@ -1213,7 +1216,7 @@ PLLM_API int pllm_paged_attention_mfma_terms(const void* q, int q_stride, const 
                                              int num_work, int single_prompt, float score_cap, const float* slopes, const float* sinks,
                                              hipStream_t stream) {
   const ScoreTerms given{score_cap, slopes, sinks};
-  if (!(score_cap >= 0.f) || (given.any() && !kTerms)) return -2;
+  if (!(score_cap >= 0.f) || (given.any() && !kTerms) || ((score_cap > 0.f || slopes) && !kForms)) return -2;
   return launch_attention(q, q_stride, k_pages, v_pages, out, out_stride, block_tables, bt_stride, cu_seqlens_q, seq_lens_k, num_seqs,
                           total_q, max_q_len, num_heads, num_kv_heads, block_size, scale, window, partition_size, num_partitions,
                           partials, waves, column_blocks, work_list, num_work, single_prompt, given, stream);

@@ -152,6 +152,102 @@ __global__ __launch_bounds__(64) void attn_prepare_kernel(
   }
 }
 
+// The same without a convolution, four successive elements per lane and L lanes per head (D <= 4 L), 256 / L heads to a workgroup:
+// everything a lane needs is asked for in a few 16-byte loads, the rotation's mate elements come from another lane's registers
+// (the pairs (i, i + rot/2), rot a multiple of 8), and the mean squares are sums over L lanes.  Where the general kernel keeps a
+// wavefront waiting for each head of 64 elements, this one has four heads in it.
+template <typename T> struct alignas(4 * sizeof(T)) PrepQuad { T v[4]; };
+
+template <typename T, int L>
+__global__ __launch_bounds__(256) void attn_prepare_quads_kernel(
+    const float* __restrict__ proj, int ld, const float* __restrict__ bias, const int* __restrict__ positions, const float* __restrict__ cos_table,
+    const float* __restrict__ sin_table, int rot, float eps, int qk_norm, int norm_first, const float* __restrict__ q_norm_w,
+    const float* __restrict__ k_norm_w, int v_mode, int heads, int kv_heads, int d, int dv, int D, int num_heads, T* __restrict__ q_out,
+    const int* __restrict__ slot_mapping, T* __restrict__ k_pages, T* __restrict__ v_pages, int block_size) {
+  const int lane = threadIdx.x % L;
+  const int tok = blockIdx.x, hs = blockIdx.y * (256 / L) + threadIdx.x / L;
+  const bool on = hs < num_heads;                              // (lanes of a head past the last only keep the others company)
+  int kind, head, base, width;
+  if (hs < heads) { kind = 0; head = hs; base = hs * d; width = d; }
+  else if (hs < heads + kv_heads) { kind = 1; head = hs - heads; base = heads * d + head * d; width = d; }
+  else if (v_mode == 2) { kind = 2; head = hs - heads - kv_heads; base = heads * d + head * d; width = d; }
+  else { kind = 2; head = hs - heads - kv_heads; base = (heads + kv_heads) * d + head * dv; width = dv; }
+  const int e = 4 * lane, half = rot >> 1;
+  const bool in = on && e < width, turns = in && kind < 2 && e < rot;
+  const bool low = e < half;
+  const float* norm_w = kind == 0 ? q_norm_w : k_norm_w;
+  const bool normed = kind < 2 ? qk_norm != 0 : v_mode == 1;
+  const bool weighed = kind < 2 && normed && norm_w;
+  float x[4] = {0.f, 0.f, 0.f, 0.f}, c[4] = {1.f, 1.f, 1.f, 1.f}, s[4] = {0.f, 0.f, 0.f, 0.f}, w[4] = {1.f, 1.f, 1.f, 1.f};
+  auto load4 = [](const float* p, float* v) {
+    const float4 q = *reinterpret_cast<const float4*>(p);
+    v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
+  };
+  const int slot = (on && kind > 0 && slot_mapping) ? slot_mapping[tok] : -1;
+  if (in) {
+    load4(proj + (size_t)tok * ld + base + e, x);
+    if (bias) {
+      float b[4];
+      load4(bias + base + e, b);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[i] += b[i];
+    }
+    if (weighed) load4(norm_w + e, w);
+  }
+  if (turns) {
+    const size_t at = (size_t)positions[tok] * half + (low ? e : e - half);
+    load4(cos_table + at, c);
+    load4(sin_table + at, s);
+  }
+  auto unit_rms = [&]() {
+    float sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) sq = fmaf(x[i], x[i], sq);      // (elements past the head are zero)
+    sq += dpp_move<kDppSwap1>(sq);
+    sq += dpp_move<kDppSwap2>(sq);
+    sq += dpp_move<kDppHalfMirror>(sq);
+    sq += dpp_move<kDppMirror>(sq);
+    if (L >= 32) sq += __shfl_xor(sq, 16);
+    if (L >= 64) sq += __shfl_xor(sq, 32);
+    const float inv = 1.f / sqrtf(sq / (float)width + eps);
+    if (normed)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[i] *= weighed ? inv * w[i] : inv;
+  };
+  if (norm_first || kind == 2) unit_rms();
+  {
+    const int mate = (threadIdx.x & 63) + (low ? half / 4 : -(half / 4));
+    float other[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) other[i] = __shfl(x[i], mate & 63);
+    if (turns)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float lo, hi;
+        if (low) rotate_pair(x[i], other[i], c[i], s[i], lo, hi); else rotate_pair(other[i], x[i], c[i], s[i], lo, hi);
+        x[i] = low ? lo : hi;
+      }
+  }
+  if (!norm_first && kind < 2) unit_rms();
+  if (!on || e >= D) return;
+  PrepQuad<T> o;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) o.v[i] = from_f32<T>(x[i]);
+  if (kind == 0) {
+    *reinterpret_cast<PrepQuad<T>*>(q_out + ((size_t)tok * heads + head) * D + e) = o;
+    return;
+  }
+  if (slot < 0) return;
+  const int page = slot / block_size, off = slot - page * block_size;
+  if (kind == 1) {
+    *reinterpret_cast<PrepQuad<T>*>(k_pages + (((size_t)page * kv_heads + head) * block_size + off) * D + e) = o;
+  } else {
+    T* out = v_pages + (((size_t)page * kv_heads + head) * D + e) * block_size + off;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) out[(size_t)i * block_size] = o.v[i];
+  }
+}
+
 // state[k] <- the projected row (with bias) of token q_len - (taps - 1) + k of this step, or what the state held for it.
 __global__ __launch_bounds__(256) void conv_inputs_keep_kernel(
     const float* __restrict__ proj, int ld, const float* __restrict__ bias, float* state, size_t slot_stride,
@@ -191,7 +287,21 @@ PLLM_API int pllm_attn_prepare(int dtype, const float* proj, int ld, const float
   if (rot > 0 && (!cos_table || !sin_table)) return -2;
   if (taps > 1 && (!conv_w || !state || !state_slots || !seq_starts || !cu_seqlens)) return -2;
   const bool write = slot_mapping && k_pages && v_pages;
-  dim3 grid(num_tokens, heads + (write ? 2 * kv_heads : 0)), block(64);
+  const int num_heads = heads + (write ? 2 * kv_heads : 0);
+  const bool quads = !conv_w && !interleaved && d % 4 == 0 && dv % 4 == 0 && D % 4 == 0 && rot % 8 == 0 && ld % 4 == 0 && (uintptr_t)proj % 16 == 0 &&
+                     (uintptr_t)bias % 16 == 0 && (uintptr_t)q_norm_w % 16 == 0 && (uintptr_t)k_norm_w % 16 == 0 &&
+                     (uintptr_t)cos_table % 16 == 0 && (uintptr_t)sin_table % 16 == 0;
+  if (quads) {
+#define PLLM_PREPQ(T, L)                                                                                                          \
+  hipLaunchKernelGGL((attn_prepare_quads_kernel<T, L>), dim3(num_tokens, (num_heads + 256 / L - 1) / (256 / L)), dim3(256), 0, stream, proj, ld, \
+                     bias, positions, cos_table, sin_table, rot, eps, qk_norm, norm_first, q_norm_w, k_norm_w, v_mode, heads, kv_heads, d, dv, D, \
+                     num_heads, (T*)q_out, slot_mapping, (T*)k_pages, (T*)v_pages, block_size)
+    if (dtype == PLLM_F32) { if (D <= 64) PLLM_PREPQ(float, 16); else if (D <= 128) PLLM_PREPQ(float, 32); else PLLM_PREPQ(float, 64); }
+    else { if (D <= 64) PLLM_PREPQ(bf16, 16); else if (D <= 128) PLLM_PREPQ(bf16, 32); else PLLM_PREPQ(bf16, 64); }
+#undef PLLM_PREPQ
+    PLLM_RETURN_LAST_ERROR();
+  }
+  dim3 grid(num_tokens, num_heads), block(64);
 #define PLLM_PREP(T)                                                                                                              \
   hipLaunchKernelGGL(attn_prepare_kernel<T>, grid, block, 0, stream, proj, ld, bias, conv_w, taps, state, (size_t)slot_stride,   \
                      state_slots, seq_starts, cu_seqlens, num_seqs, positions, cos_table, sin_table, rot, interleaved, eps, qk_norm, norm_first, \

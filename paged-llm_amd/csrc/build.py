@@ -148,8 +148,10 @@ COMMON_SOURCES = ["elementwise.hip", "gemm_generic.hip", "attention_generic.hip"
                   "selective_scan.hip", "delta_rule.hip"]
 # Head sizes whose attention library a full build makes (others are compiled at first use).
 USUAL_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 144, 160, 256)
-# ... and those whose attention library with further score terms in its loops (-DSCORE_TERMS=1) it makes as well.
+# ... and those whose attention library with further score terms in its loops (-DSCORE_TERMS=1), or with sinks alone
+# (-DSCORE_TERMS=2), it makes as well.
 SCORE_TERMS_HEAD_DIMS = (16, 32, 48, 64, 96, 128, 144)
+SINKS_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 144, 256)
 
 
 # ... and those whose attention library without a softmax (sigmoid weights) it makes.
@@ -161,6 +163,7 @@ def all_targets() -> list[tuple[str, dict]]:
     targets: list[tuple[str, dict]] = [(s, {}) for s in COMMON_SOURCES]
     targets += [("attention_mfma.hip", {"HEAD_DIM": d}) for d in USUAL_HEAD_DIMS]
     targets += [("attention_mfma.hip", {"HEAD_DIM": d, "SCORE_TERMS": 1}) for d in SCORE_TERMS_HEAD_DIMS]
+    targets += [("attention_mfma.hip", {"HEAD_DIM": d, "SCORE_TERMS": 2}) for d in SINKS_HEAD_DIMS]
     targets += [("attention_sigmoid.hip", {"HEAD_DIM": d}) for d in SIGMOID_HEAD_DIMS]
     return targets
 

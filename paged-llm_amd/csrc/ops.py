@@ -324,6 +324,10 @@ class ScoreTerms:
     def any(self) -> bool:
         return self.cap > 0.0 or self.slopes is not None or self.sinks is not None
 
+    def compiled_as(self) -> int:
+        """The form of the matrix-core kernels that serves these terms: 0 without any, 1 with all of them, 2 with sinks alone."""
+        return 1 if self.cap > 0.0 or self.slopes is not None else 2 if self.sinks is not None else 0
+
     def checked(self, num_heads: int, device) -> "ScoreTerms":
         _need(self.cap >= 0.0 and self.cap == self.cap, f"a cap of the scores is positive, or 0 for none; got {self.cap}")
         for name, t in (("slopes", self.slopes), ("sinks", self.sinks)):
@@ -929,13 +933,13 @@ def paged_attention_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.
                 _attn_scratch_retired.append(ws)
             ws = torch.empty(max(floats, 1 << 22), dtype=torch.float32, device=q.device)
             _attn_scratch[key] = ws
-    with_terms = terms is not None and terms.checked(num_heads, q.device).any()
-    defines = {"HEAD_DIM": head_dim, "SCORE_TERMS": 1} if with_terms else {"HEAD_DIM": head_dim}
+    with_terms = terms.checked(num_heads, q.device).compiled_as() if terms is not None else 0
+    defines = {"HEAD_DIM": head_dim, "SCORE_TERMS": with_terms} if with_terms else {"HEAD_DIM": head_dim}
     if (head_dim, with_terms) not in _attn_checked:   # the library on disk is the one compiled for this head size
         built = _fn("attention_mfma.hip", "pllm_attention_mfma_head_dim", defines, [])()
         _need(built == head_dim, f"attention library for head size {head_dim} reports head size {built}")
         has_terms = _fn("attention_mfma.hip", "pllm_attention_mfma_score_terms", defines, [])()
-        _need(bool(has_terms) == with_terms, f"attention library for head size {head_dim}: further score terms compiled in: {has_terms}")
+        _need(has_terms == with_terms, f"attention library for head size {head_dim}: further score terms compiled in: {has_terms}")
         _attn_checked.add((head_dim, with_terms))
     args = (_ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(block_tables),
             block_tables.stride(0), _ptr(cu_seqlens_q), _ptr(seq_lens_k), S, T, int(max_q_len), num_heads, num_kv_heads, bs,
