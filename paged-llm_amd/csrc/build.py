@@ -151,7 +151,7 @@ USUAL_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 144, 160, 256)
 # ... and those whose attention library with further score terms in its loops (-DSCORE_TERMS=1), or with sinks alone
 # (-DSCORE_TERMS=2), it makes as well.
 SCORE_TERMS_HEAD_DIMS = (16, 32, 48, 64, 96, 128, 144)
-SINKS_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 144, 256)
+SINKS_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 144, 160, 256)
 
 
 # ... and those whose attention library without a softmax (sigmoid weights) it makes.
