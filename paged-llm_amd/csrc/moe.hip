@@ -227,9 +227,10 @@ PLLM_API int pllm_moe_route(int dtype, const void* h, int ld, const float* route
   int segments = 1;
   while (segments < kRoutePieces && ((n_all + 7) / 8) * segments < kRoutePieces && width / (2 * segments) >= 64) segments *= 2;
   const size_t lds_one = (size_t)(2 * n_all + groups + segments * n_all) * sizeof(float);
-  // tokens to a workgroup (one wavefront each for the choice): 8 in steps of 512 tokens and more, 4 from 128 on, else one
-  // token to sixteen wavefronts
-  const int tok = (num_tokens >= 512 && 8 * lds_one <= 48 * 1024) ? 8 : (num_tokens >= 128 && 4 * lds_one <= 48 * 1024) ? 4 : 1;
+  // tokens to a workgroup: one, to sixteen wavefronts, while the GPU holds two such workgroups per compute unit (512 tokens of width
+  // 2,048 and 16 outputs: 21 us against 23 with eight; 256 tokens: 12 and 23), then eight (one wavefront each for the choice; 2,048
+  // tokens: 23 us against 69), or four where eight tokens' outputs do not fit
+  const int tok = num_tokens <= 512 ? 1 : 8 * lds_one <= 48 * 1024 ? 8 : 4 * lds_one <= 48 * 1024 ? 4 : 1;
   const size_t lds = lds_one * tok;
 #define PLLM_ROUTE(T, TOK, THREADS)                                                                                              \
   hipLaunchKernelGGL((moe_route_kernel<T, TOK>), dim3((num_tokens + TOK - 1) / TOK), dim3(THREADS), lds, stream, (const T*)h, ld, \

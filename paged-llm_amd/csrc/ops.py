@@ -860,7 +860,10 @@ def attention_plan(num_seqs: int, num_kv_heads: int, max_q_len: int, max_k_len: 
     if cols > 64 or max_k_len <= 64:
         return 1, 0, 1
     ncb = 1 if cols <= 16 else (2 if cols <= 32 else 4)
-    max_waves = 8
+    # Heads above 128 elements: a block of 64 keys and values takes more registers than eight wavefronts of a workgroup have
+    # (64 sequences x 1 kv head x 2048 keys, in partitions of 512: at head size 144 29.0 us with four wavefronts, 39.3 with
+    # eight; at 256 63 and 107 us).
+    max_waves = 8 if head_dim <= 128 else 4
     while max_waves >= 4 and _merge_lds_bytes(ncb, max_waves, head_dim) > lds_limit:
         max_waves //= 2
     if max_waves < 4:

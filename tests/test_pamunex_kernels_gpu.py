@@ -122,7 +122,7 @@ def test_the_layer_norm_forms_the_experts_sum_itself(width, top, dtype):
 def test_the_choice_by_the_two_largest_scores_of_a_group(n, groups, keep, top):
     from paged_llm_amd.csrc import ops
     gen = torch.Generator().manual_seed(n)
-    h = torch.randn((515 if n % 2 else 203, 40), generator=gen)                # (steps of 128 and of 512 tokens and more: four and eight tokens to a workgroup)
+    h = torch.randn((515 if n % 2 else 203, 40), generator=gen)                # (steps of up to 512 tokens and of more: one and eight tokens to a workgroup)
     w = torch.randn((n, 40), generator=gen) * 0.4
     scores = torch.sigmoid(h.double() @ w.double().T)
     want = plain.choose(scores, top, groups, keep).sort(dim=1).values
