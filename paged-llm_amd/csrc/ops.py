@@ -2166,13 +2166,15 @@ def moe_route(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor 
 
 def moe_tile_rows(pairs: int, experts: int, dtype: torch.dtype, *inner_sizes: int) -> int:
     """Rows of a tile of the experts' products for a step of ``pairs`` (token, choice) pairs: where the matrix-core
-    kernels run (bfloat16, every product's inner size a multiple of 8) 128 if an expert gets 128 pairs or more on average
-    and 64 if it gets 32 or more, else 16.  It depends on the step's number of tokens only, so a replayed step keeps its choice."""
+    kernels run (bfloat16, every product's inner size a multiple of 8) 128 if an expert gets 32 pairs or more on average, 64
+    where tiles of 128 would leave compute units idle (small experts) unless an expert gets 128; else 16.  (Both products at width
+    2,048, 30 gated experts of 1,408, 512 tokens with 4 choices: 240 us with tiles of 128, 408 with 64, 465 with 16; 16 experts of
+    1,024 at width 1,024, 256 tokens: 73, 66 and 83.)  It depends on the step's number of tokens only, so a replayed step keeps its choice."""
     if dtype == torch.bfloat16 and all(k % 8 == 0 for k in inner_sizes):
         if pairs >= 128 * experts:
             return MOE_MAX_TILE_ROWS
         if pairs >= 32 * experts:
-            return MOE_MID_TILE_ROWS
+            return MOE_MAX_TILE_ROWS if experts * max(inner_sizes[:2]) // 128 >= 160 else MOE_MID_TILE_ROWS
     return MOE_TILE_ROWS
 
 

@@ -69,3 +69,19 @@ def test_streaming_product_plans_by_sizes():
     assert plan(64, 2048, 2048, cus, partial=False) == (1, 1) and plan(64, 6144, 4096, cus, partial=False) == (2, 1)
     assert ops.gated_blocks_per_workgroup(5632, cus) == 3 and ops.gated_blocks_per_workgroup(14336, cus) == 4
     assert ops.gated_blocks_per_workgroup(8192, cus) == 4     # 1024 blocks: 342 workgroups of three would need a second round
+
+
+def test_tiles_of_the_experts_products_by_sizes():
+    import torch
+    from paged_llm_amd.csrc import ops
+    rows = lambda tokens, top, experts, width, ff, dtype=torch.bfloat16: ops.moe_tile_rows(tokens * top, experts, dtype, width, ff, width)
+    assert rows(64, 4, 16, 2048, 2048) == 16 and rows(127, 4, 16, 2048, 2048) == 16      # fewer than 32 pairs an expert
+    assert rows(128, 4, 16, 2048, 2048) == 128 and rows(2048, 4, 16, 1024, 1024) == 128
+    assert rows(256, 4, 16, 1024, 1024) == 64 and rows(512, 4, 16, 1024, 1024) == 128    # small experts: tiles that reach every compute unit
+    assert rows(2048, 4, 16, 2048, 2048, torch.float32) == 16 and rows(2048, 4, 16, 50, 2048) == 16      # the plain kernel's tiles
+
+
+def test_decode_attention_of_large_heads_keeps_to_four_wavefronts():
+    for d in (144, 160, 256):
+        assert ops.attention_plan(64, 1, 1, 2048, 16, d, 160 * 1024) == (4, 512, 4)
+    assert ops.attention_plan(64, 1, 1, 2048, 16, 128, 160 * 1024) == (8, 512, 4)
